@@ -374,14 +374,28 @@ enum {
     ZG_LM_MIX_GLA = 6,              /* gated linear attention with a decay per key channel: q = W_q h / sqrt(dim), k, v, gate plain
                                        projections; f = sigmoid(W_a2 W_a1 h + b_a)^(1 / tau);  S = diag(f) S + k v^T;  o = S^T q;
                                        every head's o RMS-normed over vdim with one plain weight [vdim], times silu(W_g h), then W_o */
-    ZG_LM_MIX_ATTENTION = 7         /* causal grouped-query softmax attention over the whole sequence, no rotation, no value
+    ZG_LM_MIX_ATTENTION = 7,        /* causal grouped-query softmax attention over the whole sequence, no rotation, no value
                                        projection: the VALUE of a key head is that head's un-normalised key; q and k are divided by their
                                        root mean square per head (no weight); the query of position p is multiplied by
                                        1 + qtemp_coef ln(floor((p + 1) / qtemp_every) + 1) (qtemp_every 0: not);
                                        score = scale q . k, then softcap tanh(score / softcap) (softcap 0: not), then minus
                                        2^(-8 (h + 1) / heads) (i - j) for head h (dist_bias 0: not) */
+    ZG_LM_MIX_ROTARY_ATTENTION = 8, /* causal grouped-query softmax attention with rotary positions on the first rot_dims channels of q
+                                       and k (any pairing, scaled frequencies and amplitude allowed); with chunk > 0 a query sees the keys
+                                       of its own chunk of positions [n chunk, (n + 1) chunk) only, with window > 0 those of its window */
+    ZG_LM_MIX_SSD = 9               /* selective state space with a scalar decay per head and token (Mamba-2): in = [z (heads vdim) |
+                                       x (heads vdim) | B (kv_heads dim) | C (kv_heads dim) | dt (heads)] rows of one projection; x, B, C
+                                       pass a causal convolution of `conv` taps with bias and silu; dt = softplus(dt + dt_bias);
+                                       S = exp(-exp(A_log) dt) S + dt B x^T ([dim][vdim] per head, B and C shared by heads / kv_heads
+                                       heads); y = S^T C + D x; y silu(z) RMS-normed in norm_groups equal parts, times a plain weight */
 };
-enum { ZG_LM_FF_NONE = 0, ZG_LM_FF_DENSE = 1 /* down(relu(up h)^2) */, ZG_LM_FF_MOE = 2 /* top-k of `experts` units */ };
+enum { ZG_LM_FF_NONE = 0, ZG_LM_FF_DENSE = 1 /* down(act(up h)) */, ZG_LM_FF_MOE = 2 /* top-k of `experts` units */ };
+/* Activation of the dense feed-forward (dense_act). */
+enum {
+    ZG_LM_DENSE_RELU2 = 0,   /* relu(z)^2 */
+    ZG_LM_DENSE_POLYNORM = 1 /* a N(z) + b N(z^2) + c N(z^3) + e, N(v) = v / sqrt(mean(v^2) + norm_eps) over the row; the fp32 tensor
+                                `mlp.act` holds a, b, c, e */
+};
 /* Activation of an expert (ff_act) and the rule of the router (router) of ZG_LM_FF_MOE. */
 enum {
     ZG_LM_ACT_GLU_SILU = 0, /* down(silu(gate h) * up h): tensors e<j>.gate / up / down */
@@ -402,9 +416,10 @@ enum { ZG_LM_ROT_PLAIN = 0, ZG_LM_ROT_YARN = 1 /* blend by pair index, amplitude
 typedef struct {
     int mixer;                    /* ZG_LM_MIX_* */
     int heads, dim, vdim;         /* both mixers: heads, key (unrotated) channels and value channels per head */
-    int rot_dim, kv_rank, q_rank; /* latent attention: rotated channels per head, latent sizes of keys/values and of queries */
+    int rot_dim, kv_rank, q_rank; /* latent attention: rotated channels per head, latent sizes of keys/values and of queries (q_rank 0: the
+                                     queries are projected directly, tensor `mix.q`) */
     float scale;                  /* latent attention: factor of the scores */
-    int rot_dims;                 /* rotary: how many of the rot_dim channels are rotated (interleaved pairs) */
+    int rot_dims;                 /* rotary: how many of the rot_dim channels are rotated */
     float rot_base;
     int rot_scaled;               /* ZG_LM_ROT_*: YARN blends the frequencies with the four constants below; BANDS keeps a frequency whose
                                      wavelength is below original / rot_fast, divides it by factor above original / rot_slow, and
@@ -438,6 +453,14 @@ typedef struct {
     float route_scale;            /* ZG_LM_ROUTE_SIGMOID_GROUPS: factor of the normalised weights (0: 1) */
     int weights_of;               /* > 0: this layer owns no tensors and runs those of layer weights_of - 1 (whose other fields it
                                      repeats) with separate cache and state */
+    int rot_halves;               /* != 0: rotary pairs are the channels (i, i + rot_dims / 2), 0: (2i, 2i + 1) */
+    int chunk;                    /* rotary attention: > 0: a position sees only its own chunk of this many positions, counted from the start
+                                     of the sequence */
+    int kv_from;                  /* latent attention: > 0: no latents of its own; it reads those that layer kv_from - 1 (in front of it, with
+                                     the same kv_rank, rot_dim and rotation) has cached */
+    int head_gate;                /* latent attention: != 0: head h's output is multiplied by sigmoid(W_g h)_h (tensor `mix.g`) */
+    int norm_groups;              /* selective state space: equal parts of the norm behind the gate (0: 1) */
+    int dense_act;                /* ZG_LM_DENSE_* */
 } zg_lm_layer;
 enum {
     ZG_LM_F32 = 1 << 0,     /* true 32-bit products everywhere */
@@ -453,7 +476,9 @@ enum {
                                   is reduced over the row — with the scalar `<name>.alpha` and the vector `<name>.b` beside the weight `<name>`; the
                                   mixer reads norm1(x) as it is (no token shift, no input convolution), and a sublayer's normed output
                                   enters the residual sum times residual_mult */
-    ZG_LM_EMBED_NORM = 1 << 7  /* the embedding output passes the stack's norm with the tensors `embed.norm` (ZG_LM_TANH_NORMS only) */
+    ZG_LM_EMBED_NORM = 1 << 7, /* the embedding output passes the stack's norm with the tensors `embed.norm` (ZG_LM_TANH_NORMS only) */
+    ZG_LM_NO_SHIFT = 1 << 8    /* sequential sublayers with RMS norms whose mixer reads norm1(x) as it is: no token shift, no input
+                                  convolution */
 };
 typedef struct {
     size_t vocab, width, n_layers;
@@ -483,8 +508,10 @@ int zg_lm_destroy(zg_lm* g);
  * left.v left.sink left.talk left.o left.out right.y right.y.b right.x right.x.b right.conv right.conv.b right.ra right.ra.b
  * right.ri right.ri.b right.lam right.o right.out; delta rule: q q.conv k k.conv v v.conv b A_log dt_bias a1 a2 g1 g2 norm o;
  * window + linear pair: left.q|k|v with .b and .conv each, left.q.norm left.k.norm left.g left.o left.o.b right.q right.k right.v
- * right.g right.norm right.o right.decay; gated linear attention: q k v g o norm a1 a2 a2.b; attention: q k o)
- * and `l<i>.mlp.*` (dense: up down; experts: e<j>.gate e<j>.up e<j>.down router, and correction or router.b; shared.gate shared.up
+ * right.g right.norm right.o right.decay; gated linear attention: q k v g o norm a1 a2 a2.b; attention: q k o;
+ * rotary attention: q k v o; selective state space: in conv conv.b dt_bias A_log D norm o; latent attention with q_rank 0: q for
+ * dq dq.norm uq, with head_gate also g, with kv_from no dkv and dkv.norm)
+ * and `l<i>.mlp.*` (dense: up down, and act with a polynomial activation; experts: e<j>.gate e<j>.up e<j>.down router, and correction or router.b; shared.gate shared.up
  * shared.down shared.sg).  data: fp32 on the host, `len` elements, matrices
  * [out][in] row-major; matrices are stored bf16 (round to nearest even).  ZG_ERR_ARG for a name the configuration does not have. */
 int zg_lm_load_tensor(zg_lm* g, const char* name, const float* data, size_t len);

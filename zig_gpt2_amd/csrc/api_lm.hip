@@ -29,6 +29,10 @@
 // with separate cache and state.  Their gated linear attention keeps its [heads][dim][vdim] state in the block of sequence
 // state; their attention caches the normed key heads and, as values, the projected ones.
 //
+// A selective state space keeps the tail of its convolution and its [heads][state][vdim] state in the block of sequence state; chunked
+// attention caches rotated keys and plain values like the windowed one (a chunk is a window whose front edge moves by whole chunks).
+// A latent attention layer may read the latents another layer has cached: it then owns no cache, and its pass points at that one's.
+//
 // Latent attention runs in its absorbed form in prompts and in decoding alike: score_j = (W_uk^T q_nope) . c_j + q_rot . k_rot_j,
 // out = W_uv (sum_j p_j c_j) — only the latent c_j and the rotated key part are cached, and a portion of a prompt needs nothing
 // of the tokens before it but their cache rows.
@@ -90,6 +94,9 @@ struct LayerW {
     float *qkv_bias = nullptr, *qnorm = nullptr, *knorm = nullptr, *rnorm = nullptr, *obias = nullptr, *decay = nullptr;
     // gated linear attention: the bias of the decay's second step;  attention: the heads' slopes of the distance bias
     float *a2b = nullptr, *slopes = nullptr;
+    // selective state space: the skip factors and the weight of the norm in parts;  polynomial activation: its four numbers
+    float *skip = nullptr, *part_norm = nullptr, *poly = nullptr;
+    int ld_cat = 0;  // row stride of the fused projection's output (a multiple of four: 16-byte loads behind it)
 };
 
 struct Pass {
@@ -196,6 +203,7 @@ struct zg_lm {
     int keep_pages = 0;   // pages that hold those first tokens: never returned while the sequence is open
     float embed_scale = 1.0f;
     bool side = false;          // ZG_LM_SIDE_BY_SIDE
+    bool no_shift = false;      // ZG_LM_NO_SHIFT
     bool tanh_norms = false;    // ZG_LM_TANH_NORMS: every norm pointer is a block [w | b | alpha]
     float res_mult = 1.0f;      // ... and a sublayer's normed output enters the residual sum times this
     float* embed_norm = nullptr;  // ZG_LM_EMBED_NORM
@@ -237,6 +245,12 @@ namespace {
 // ids | pos | slot | prev | last-entry | want rows | entry start | entry len | entry slot | place of the row inside its entry
 size_t meta_ints(const zg_lm* g) { return (size_t)7 * g->MS + (size_t)3 * g->NS; }
 size_t meta_row_off(const zg_lm* g) { return (size_t)6 * g->MS + (size_t)3 * g->NS; }
+
+// The most keys a row of a rotary attention layer can see.
+int rotary_key_capacity(const zg_lm* g, const zg_lm_layer& d) {
+    const int all_keys = g->max_pages * g->P;
+    return d.chunk > 0 ? std::min(d.chunk, all_keys) : d.window > 0 ? std::min(d.window, all_keys) : all_keys;
+}
 
 // Everything that lives in the arena, in one place: called once with a null base to measure and once to place.
 void layout(zg_lm* g, Bump& b) {
@@ -316,7 +330,8 @@ void layout(zg_lm* g, Bump& b) {
         if (g->side || tn) {
         } else {
             vec(p + "norm1b", L.norm1b, W, INIT_OFFSET);
-            if (taps == 0) vec(p + "shift", L.shift, W, INIT_UNIT);
+            if (g->no_shift) {
+            } else if (taps == 0) vec(p + "shift", L.shift, W, INIT_UNIT);
             else vec(p + "canon1", L.canon1, W * taps, INIT_OFFSET);
         }
         const size_t H = d.heads, D = d.dim, Vd = d.vdim;
@@ -457,6 +472,40 @@ void layout(zg_lm* g, Bump& b) {
             const int cap = g->max_pages * g->P;
             max_win = std::max(max_win, std::min(window_split_workspace((int)MS, (int)H, (int)D, cap, nullptr), (size_t)1 << 29));
             max_win_few = std::max(max_win_few, window_split_workspace(kGemvMaxRows, (int)H, (int)D, cap, nullptr));
+        } else if (d.mixer == ZG_LM_MIX_ROTARY_ATTENTION) {
+            const size_t G = d.kv_heads, HD = H * D, GD = G * D, GV = G * Vd, NP = HD + GD + GV;
+            L.n_cat = (int)NP;
+            L.ld_cat = (int)((NP + 3) & ~(size_t)3);
+            L.wcat = b.take<bf16_t>(NP * W);  // q | k | v
+            mat(p + "mix.q", L.wcat, 0, HD, W);
+            mat(p + "mix.k", L.wcat, HD, GD, W);
+            mat(p + "mix.v", L.wcat, HD + GD, GV, W);
+            L.o = b.take<bf16_t>(W * H * Vd);
+            mat(p + "mix.o", L.o, 0, W, H * Vd);
+            L.rot_freq = b.take<float>(std::max<size_t>(1, d.rot_dims / 2));
+            max_proj = std::max(max_proj, (size_t)L.ld_cat);
+            max_o = std::max(max_o, H * Vd);
+            const int cap = rotary_key_capacity(g, d);
+            max_win = std::max(max_win, std::min(window_split_workspace((int)MS, (int)H, (int)Vd, cap, nullptr), (size_t)1 << 29));
+            max_win_few = std::max(max_win_few, window_split_workspace(kGemvMaxRows, (int)H, (int)Vd, cap, nullptr));
+        } else if (d.mixer == ZG_LM_MIX_SSD) {
+            const size_t G = d.kv_heads, HV = H * Vd, CC = HV + 2 * G * D, NP = HV + CC + H;
+            L.n_cat = (int)NP;
+            L.ld_cat = (int)((NP + 3) & ~(size_t)3);
+            L.wcat = b.take<bf16_t>(NP * W);  // z | x | B | C | dt, one tensor
+            mat(p + "mix.in", L.wcat, 0, NP, W);
+            vec(p + "mix.conv", L.convw, CC * d.conv, INIT_OFFSET);
+            vec(p + "mix.conv.b", L.convb, CC, INIT_OFFSET);
+            vec(p + "mix.dt_bias", L.dt_bias, H, INIT_OFFSET);
+            vec(p + "mix.A_log", L.a_log, H, INIT_OFFSET);
+            vec(p + "mix.D", L.skip, H, INIT_PLAIN);
+            vec(p + "mix.norm", L.part_norm, HV, INIT_PLAIN);
+            L.o = b.take<bf16_t>(W * HV);
+            mat(p + "mix.o", L.o, 0, W, HV);
+            max_proj = std::max(max_proj, (size_t)L.ld_cat);
+            max_o = std::max(max_o, HV);
+            max_t = std::max(max_t, CC);
+            max_scan = std::max(max_scan, HV * D + H);
         } else if (d.mixer == ZG_LM_MIX_HGRN2) {
             const size_t HD = H * D, HV = H * Vd;
             L.qfv = b.take<bf16_t>((2 * HD + HV) * W);
@@ -472,14 +521,22 @@ void layout(zg_lm* g, Bump& b) {
             max_scan = std::max(max_scan, H * D * Vd + H * D);
             max_o = std::max(max_o, HV);
         } else {
-            const size_t R = d.rot_dim, KR = d.kv_rank, QR = d.q_rank, HV = H * Vd;
-            L.dqkv = b.take<bf16_t>((QR + KR + R) * W);
-            mat(p + "mix.dq", L.dqkv, 0, QR, W);
-            mat(p + "mix.dkv", L.dqkv, QR, KR + R, W);
-            vec(p + "mix.dq.norm", L.dq_norm, QR, INIT_PLAIN);
-            vec(p + "mix.dkv.norm", L.dkv_norm, KR, INIT_PLAIN);
-            L.uq = b.take<bf16_t>(H * (D + R) * QR);
-            mat(p + "mix.uq", L.uq, 0, H * (D + R), QR);
+            const size_t R = d.rot_dim, KR = d.kv_rank, QR = d.q_rank, HV = H * Vd, NG = d.head_gate ? H : 0, NL = d.kv_from > 0 ? 0 : KR + R;
+            const size_t NQ = QR > 0 ? QR : H * (D + R), NP = NQ + NL + NG;  // dq, or q itself | dkv | gate
+            L.n_cat = (int)NP;
+            L.ld_cat = QR > 0 && NG == 0 ? (int)NP : (int)((NP + 3) & ~(size_t)3);
+            L.dqkv = b.take<bf16_t>(NP * W);
+            mat(p + (QR > 0 ? "mix.dq" : "mix.q"), L.dqkv, 0, NQ, W);
+            if (NL) {
+                mat(p + "mix.dkv", L.dqkv, NQ, NL, W);
+                vec(p + "mix.dkv.norm", L.dkv_norm, KR, INIT_PLAIN);
+            }
+            if (NG) mat(p + "mix.g", L.dqkv, NQ + NL, NG, W);
+            if (QR > 0) {
+                vec(p + "mix.dq.norm", L.dq_norm, QR, INIT_PLAIN);
+                L.uq = b.take<bf16_t>(H * (D + R) * QR);
+                mat(p + "mix.uq", L.uq, 0, H * (D + R), QR);
+            }
             L.ukT = b.take<bf16_t>(H * KR * D);
             mat(p + "mix.uk", L.ukT, 0, H * D, KR, (int)H);
             L.uv = b.take<bf16_t>(HV * KR);
@@ -487,9 +544,9 @@ void layout(zg_lm* g, Bump& b) {
             L.o = b.take<bf16_t>(W * HV);
             mat(p + "mix.o", L.o, 0, W, HV);
             L.rot_freq = b.take<float>(std::max<size_t>(1, d.rot_dims / 2));
-            max_proj = std::max(max_proj, QR + KR + R);
+            max_proj = std::max(max_proj, (size_t)L.ld_cat);
             max_qr = std::max(max_qr, QR);
-            max_q = std::max(max_q, H * (D + R));
+            if (QR > 0) max_q = std::max(max_q, H * (D + R));
             max_qa = std::max(max_qa, H * (KR + R));
             max_ctx = std::max(max_ctx, H * KR);
             max_att_part = std::max(max_att_part, H * (KR + 2));
@@ -509,6 +566,7 @@ void layout(zg_lm* g, Bump& b) {
             mat(p + "mlp.up", L.up, 0, F, W);
             L.down = b.take<bf16_t>(W * F);
             mat(p + "mlp.down", L.down, 0, W, F);
+            if (d.dense_act == ZG_LM_DENSE_POLYNORM) vec(p + "mlp.act", L.poly, 4, INIT_PLAIN);
             max_ff = std::max(max_ff, F);
         } else if (d.ff == ZG_LM_FF_MOE) {
             const size_t E = d.experts, UF = d.ff_act == ZG_LM_ACT_GELU ? F : 2 * F;  // rows of an expert's first matrix
@@ -581,15 +639,24 @@ void layout(zg_lm* g, Bump& b) {
         } else if (d.mixer == ZG_LM_MIX_GLA) {
             ps.rec_off = sq;
             sq += (size_t)d.heads * d.dim * d.vdim;
+        } else if (d.mixer == ZG_LM_MIX_SSD) {
+            ps.conv_off = sq;
+            sq += (size_t)(d.conv - 1) * ((size_t)d.heads * d.vdim + 2 * (size_t)d.kv_heads * d.dim);
+            ps.rec_off = sq;
+            sq += (size_t)d.heads * d.dim * d.vdim;
         }
     }
     g->seq_floats = sq;
     g->seq_state = b.take<float>(std::max<size_t>(1, NS * sq));
     g->page_table = b.take<int>(NS * g->max_pages);
-    for (Pass& ps : g->passes) {
+    for (size_t pi = 0; pi < g->passes.size(); ++pi) {
+        Pass& ps = g->passes[pi];
         const zg_lm_layer& d = g->layers[ps.layer].d;
-        if (d.mixer == ZG_LM_MIX_LATENT_ATTENTION) ps.cache = b.take<float>((size_t)g->n_pages * g->P * (d.kv_rank + d.rot_dim));
-        if (d.mixer == ZG_LM_MIX_PARALLEL || d.mixer == ZG_LM_MIX_WINDOW_LINEAR)
+        if (d.mixer == ZG_LM_MIX_LATENT_ATTENTION && d.kv_from > 0) {  // the cache of the latest pass of the layer it names
+            for (size_t q = 0; q < pi; ++q)
+                if (g->passes[q].layer == d.kv_from - 1) ps.cache = g->passes[q].cache;
+        } else if (d.mixer == ZG_LM_MIX_LATENT_ATTENTION) ps.cache = b.take<float>((size_t)g->n_pages * g->P * (d.kv_rank + d.rot_dim));
+        if (d.mixer == ZG_LM_MIX_PARALLEL || d.mixer == ZG_LM_MIX_WINDOW_LINEAR || d.mixer == ZG_LM_MIX_ROTARY_ATTENTION)
             ps.cache = b.take<float>((size_t)g->n_pages * g->P * d.kv_heads * (d.dim + d.vdim));
         if (d.mixer == ZG_LM_MIX_ATTENTION) ps.cache = b.take<float>((size_t)g->n_pages * g->P * d.kv_heads * 2 * d.dim);
     }
@@ -682,9 +749,10 @@ void rotary_table(const zg_lm_layer& d, std::vector<float>& freq, float& amp) {
 }
 
 int check_layer(const zg_lm_layer& d, size_t i, unsigned flags) {
-    ZG_REQUIRE(d.mixer >= ZG_LM_MIX_HGRN2 && d.mixer <= ZG_LM_MIX_ATTENTION, ZG_ERR_ARG, "layer %zu: unknown mixer %d", i, d.mixer);
+    ZG_REQUIRE(d.mixer >= ZG_LM_MIX_HGRN2 && d.mixer <= ZG_LM_MIX_SSD, ZG_ERR_ARG, "layer %zu: unknown mixer %d", i, d.mixer);
     ZG_REQUIRE(d.heads >= 1 && d.dim >= 1 && d.vdim >= 1, ZG_ERR_ARG, "layer %zu: heads %d dim %d vdim %d", i, d.heads, d.dim, d.vdim);
-    if (d.mixer == ZG_LM_MIX_PARALLEL || d.mixer == ZG_LM_MIX_CHANNEL_DELTA || d.mixer == ZG_LM_MIX_WINDOW_LINEAR || d.mixer == ZG_LM_MIX_ATTENTION)
+    if (d.mixer == ZG_LM_MIX_PARALLEL || d.mixer == ZG_LM_MIX_CHANNEL_DELTA || d.mixer == ZG_LM_MIX_WINDOW_LINEAR || d.mixer == ZG_LM_MIX_ATTENTION ||
+        d.mixer == ZG_LM_MIX_ROTARY_ATTENTION || d.mixer == ZG_LM_MIX_SSD)
         ZG_REQUIRE(d.kv_heads >= 1 && d.heads % d.kv_heads == 0, ZG_ERR_ARG, "layer %zu: %d heads on %d key heads", i, d.heads, d.kv_heads);
     if (d.mixer == ZG_LM_MIX_PARALLEL) {
         ZG_REQUIRE(d.vdim % 2 == 0, ZG_ERR_ARG, "layer %zu: %d value channels per head cannot be rotated in pairs", i, d.vdim);
@@ -718,8 +786,18 @@ int check_layer(const zg_lm_layer& d, size_t i, unsigned flags) {
                    d.dim);
         ZG_REQUIRE(d.softcap >= 0.0f && d.qtemp_every >= 0 && d.window == 0, ZG_ERR_ARG, "layer %zu: score cap %g, query factor every %d, window %d", i,
                    d.softcap, d.qtemp_every, d.window);
+    } else if (d.mixer == ZG_LM_MIX_ROTARY_ATTENTION) {
+        ZG_REQUIRE(d.rot_dims >= 0 && d.rot_dims % 2 == 0 && d.rot_dims <= d.dim && (d.rot_dims == 0 || d.rot_base > 0.0f), ZG_ERR_ARG,
+                   "layer %zu: %d rotated dimensions of %d, base %f", i, d.rot_dims, d.dim, d.rot_base);
+        ZG_REQUIRE(d.chunk >= 0 && d.window >= 0 && (d.chunk == 0 || d.window == 0), ZG_ERR_ARG, "layer %zu: chunk %d, window %d", i, d.chunk, d.window);
+        ZG_REQUIRE(!d.rot_scaled || (d.rot_factor > 0.0f && d.rot_original > 0.0f && d.rot_fast > 0.0f && d.rot_slow > 0.0f), ZG_ERR_ARG,
+                   "layer %zu: rotary scaling constants must be positive", i);
+    } else if (d.mixer == ZG_LM_MIX_SSD) {
+        ZG_REQUIRE(d.conv >= 1 && d.conv <= 16 && d.norm_groups >= 0 && (d.heads * d.vdim) % std::max(1, d.norm_groups) == 0, ZG_ERR_ARG,
+                   "layer %zu: %d taps, %d channels normed in %d parts", i, d.conv, d.heads * d.vdim, d.norm_groups);
+        ZG_REQUIRE(d.dim <= kSsdMaxState, ZG_ERR_UNSUPPORTED, "layer %zu: a state of %d rows per head (at most %d)", i, d.dim, kSsdMaxState);
     } else {
-        ZG_REQUIRE(d.rot_dim >= 0 && d.kv_rank >= 1 && d.q_rank >= 1, ZG_ERR_ARG, "layer %zu: rot_dim %d kv_rank %d q_rank %d", i, d.rot_dim,
+        ZG_REQUIRE(d.rot_dim >= 0 && d.kv_rank >= 1 && d.q_rank >= 0 && d.kv_from >= 0, ZG_ERR_ARG, "layer %zu: rot_dim %d kv_rank %d q_rank %d", i, d.rot_dim,
                    d.kv_rank, d.q_rank);
         ZG_REQUIRE(d.rot_dims >= 0 && d.rot_dims % 2 == 0 && d.rot_dims <= d.rot_dim, ZG_ERR_ARG, "layer %zu: %d rotated dimensions of %d", i,
                    d.rot_dims, d.rot_dim);
@@ -730,6 +808,11 @@ int check_layer(const zg_lm_layer& d, size_t i, unsigned flags) {
                    "layer %zu: rotary scaling constants must be positive", i);
     }
     ZG_REQUIRE(d.ff == ZG_LM_FF_NONE || d.ff == ZG_LM_FF_DENSE || d.ff == ZG_LM_FF_MOE, ZG_ERR_ARG, "layer %zu: unknown feed-forward %d", i, d.ff);
+    ZG_REQUIRE(d.dense_act == ZG_LM_DENSE_RELU2 || d.dense_act == ZG_LM_DENSE_POLYNORM, ZG_ERR_ARG, "layer %zu: dense activation %d", i, d.dense_act);
+    ZG_REQUIRE(d.kv_from == 0 || (d.mixer == ZG_LM_MIX_LATENT_ATTENTION && d.q_rank == 0), ZG_ERR_UNSUPPORTED,
+               "layer %zu: another layer's latents are read by latent attention with directly projected queries", i);
+    ZG_REQUIRE(d.head_gate == 0 || (d.mixer == ZG_LM_MIX_LATENT_ATTENTION && d.q_rank == 0), ZG_ERR_UNSUPPORTED,
+               "layer %zu: the gate per head is built for latent attention with directly projected queries", i);
     ZG_REQUIRE(d.ff == ZG_LM_FF_NONE || d.ff_width >= 1, ZG_ERR_ARG, "layer %zu: feed-forward width %d", i, d.ff_width);
     ZG_REQUIRE(d.ff != ZG_LM_FF_MOE || (d.experts >= 1 && d.experts <= 256 && d.top >= 1 && d.top <= d.experts), ZG_ERR_UNSUPPORTED,
                "layer %zu: %d experts, %d chosen (at most 256 experts)", i, d.experts, d.top);
@@ -789,6 +872,23 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
         c.tail = g->seq_state + off; c.slot_stride = g->seq_floats;
         return launch_causal_conv(c, M, n_ent, single, d_off, d_slot, d_estart, d_elen, d_eslot, s);
     };
+    // rows of the score workspace of whole-context attention: as long as the longest sequence of this portion (a captured decode step
+    // replays at any length of its bucket, so it takes the bucket's or the cache's capacity)
+    auto whole_context_keys = [&](bool replayed) {
+        const int all_keys = g->max_pages * g->P;
+        return replayed ? (g->bucket_keys > 0 ? g->bucket_keys : all_keys) : std::min(all_keys, (g->step_keys + 63) / 64 * 64);
+    };
+    // the dense feed-forward of a layer: in -> out
+    auto dense_ff = [&](const LayerW& L, const float* in, float* out) -> int {
+        const int F = L.d.ff_width;
+        const bool poly = L.d.dense_act == ZG_LM_DENSE_POLYNORM;
+        Linear up, dn;
+        up.A = in; up.lda = W; up.B = L.up; up.ldb = W; up.C = g->u; up.ldc = F; up.M = M; up.N = F; up.K = W; up.act = poly ? ACT_NONE : ACT_RELU2;
+        ZG_TRY(launch_linear(up, f32, s));
+        if (poly) ZG_TRY(launch_polynorm(g->u, F, F, M, L.poly, eps, s));
+        dn.A = g->u; dn.lda = F; dn.B = L.down; dn.ldb = F; dn.C = out; dn.ldc = W; dn.M = M; dn.N = W; dn.K = F;
+        return launch_linear(dn, f32, s);
+    };
     bool h_ready = false;  // g->h already holds this pass's shifted norm (written by the previous pass's fused tail)
     if (tnorm) {  // the norm behind the embedding (in place) and the first pass's norm; every later one rides behind a sublayer's sum
         ZG_TRY(launch_tanh_norm(g->x, g->embed_norm, g->layers[g->passes[0].layer].norm1, nullptr, g->h, M, W, s));
@@ -811,23 +911,72 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
         if (ps.readd && !hc_ready) ZG_TRY(launch_add_rows(g->x, g->x0, M, W, s));
         if (!h_ready && !hc_ready)
             ZG_TRY(launch_norm_shift(g->x, L.norm1, canon ? nullptr : L.shift, eps, g->h, M, W, d_prev, d_slot, g->shift_state + (size_t)p * W,
-                                     (size_t)g->n_passes * W, canon ? nullptr : d_last, g->last_h + (size_t)p * NS * W, s));
+                                     (size_t)g->n_passes * W, canon || g->no_shift ? nullptr : d_last, g->last_h + (size_t)p * NS * W, s));
         h_ready = false;
         const float* hin = g->h;  // what the sublayer reads
         if (canon) {
             if (!hc_ready) ZG_TRY(input_conv(L.canon1, ps.canon1_off));
             hin = g->hc;
         }
-        // one row per entry: the pass's last sum is fused with the next pass's norm + shift (tail below)
+        // the pass's last sum fused with the next pass's norm (with a token shift: in steps of one row per entry)
         auto tail = [&](const float* y, const float* yexp, const float* weight, int top, const float* wb) -> int {
-            if (!single || p + 1 >= g->n_passes || canon) return ZG_OK;
+            if (p + 1 >= g->n_passes || canon || g->passes[p + 1].readd) return ZG_OK;
             const LayerW& N = g->layers[g->passes[p + 1].layer];
+            if (g->no_shift && y) {  // nothing of the token before: the same fusion at any number of rows
+                ZG_TRY(launch_norm_add_norm(g->x, y, wb, N.norm1, eps, g->h, M, W, s));
+                h_ready = true;
+                return ZG_OK;
+            }
+            if (!single || g->no_shift) return ZG_OK;
             return launch_sum_norm_shift(g->x, y, yexp, weight, top, wb, N.norm1, N.shift, eps, g->h, M, W, d_slot, g->shift_state + (size_t)(p + 1) * W,
                                          (size_t)g->n_passes * W, d_last, g->last_h + (size_t)(p + 1) * NS * W, s, &h_ready);
         };
         Linear lin;
         bool mid_done = false;  // x, and the feed-forward's input in g->hc, are already there
-        if (d.mixer == ZG_LM_MIX_WINDOW_LINEAR) {
+        if (d.mixer == ZG_LM_MIX_ROTARY_ATTENTION) {
+            const int G = d.kv_heads, HV = H * Vd, LD = L.ld_cat;
+            const Rotary rot{L.rot_freq, d.rot_dims, L.rot_amp, d.rot_halves};
+            KeyMask mask;
+            mask.window = d.window;
+            mask.chunk = d.chunk;
+            lin.A = hin; lin.lda = W; lin.B = L.wcat; lin.ldb = W; lin.C = g->proj; lin.ldc = LD; lin.M = M; lin.N = L.n_cat; lin.K = W;
+            ZG_TRY(launch_linear(lin, f32, s));
+            ZG_TRY(launch_window_prep(g->proj, LD, M, H, G, D, Vd, rot, nullptr, d_pos, d_slot, g->page_table, g->max_pages, g->P, ps.cache, s));
+            const int cap = rotary_key_capacity(g, d);
+            // (a bounded layer's decode steps take its bound at any length)
+            const int key_cap = (d.chunk > 0 || d.window > 0) && (single || capturing) ? cap : std::min(cap, whole_context_keys(single || capturing));
+            bool split = false;
+            ZG_TRY(launch_window_attention_split(g->proj, LD, g->o, HV, M, H, G, D, Vd, d.scale, mask, nullptr, nullptr, nullptr, d_pos, d_slot,
+                                                 g->page_table, g->max_pages, g->P, ps.cache, key_cap, g->win_ws, g->win_ws_floats, d_estart, d_elen,
+                                                 n_ent, s, &split));
+            if (!split)
+                ZG_TRY(launch_window_attention(g->proj, LD, g->o, HV, M, H, G, D, Vd, d.scale, mask, nullptr, nullptr, nullptr, d_pos, d_slot,
+                                               g->page_table, g->max_pages, g->P, ps.cache, s));
+            lin = Linear();
+            lin.A = g->o; lin.lda = HV; lin.B = L.o; lin.ldb = HV; lin.C = g->y; lin.ldc = W; lin.M = M; lin.N = W; lin.K = HV;
+            ZG_TRY(launch_linear(lin, f32, s));
+        } else if (d.mixer == ZG_LM_MIX_SSD) {
+            const int G = d.kv_heads, HV = H * Vd, CC = HV + 2 * G * D, LD = L.ld_cat;
+            lin.A = hin; lin.lda = W; lin.B = L.wcat; lin.ldb = W; lin.C = g->proj; lin.ldc = LD; lin.M = M; lin.N = L.n_cat; lin.K = W;
+            ZG_TRY(launch_linear(lin, f32, s));
+            ConvArgs cv;
+            cv.in = g->proj + HV; cv.ld_in = LD; cv.out = g->ta; cv.ld_out = CC; cv.C = CC; cv.taps = d.conv; cv.w = L.convw; cv.bias = L.convb;
+            cv.flags = CONV_SILU; cv.tail = g->seq_state + ps.conv_off; cv.slot_stride = g->seq_floats;
+            SsdArgs sa;
+            sa.z = g->proj; sa.dt = g->proj + HV + CC; sa.ld_proj = LD; sa.dt_bias = L.dt_bias; sa.a_log = L.a_log; sa.skip = L.skip;
+            sa.H = H; sa.G = G; sa.N = D; sa.V = Vd; sa.out = g->o; sa.ldo = HV; sa.state = g->seq_state + ps.rec_off; sa.slot_stride = g->seq_floats;
+            if (single) {  // decode steps: the convolution inside the scan, its tail moved on by the norm's launch
+                sa.xbc = cv.in; sa.ld_xbc = LD;
+            } else {
+                ZG_TRY(launch_causal_conv(cv, M, n_ent, false, d_off, d_slot, d_estart, d_elen, d_eslot, s));
+                sa.xbc = g->ta; sa.ld_xbc = CC;
+            }
+            ZG_TRY(launch_ssd_scan(sa, single ? &cv : nullptr, M, d_estart, d_elen, d_eslot, n_ent, g->scan_ws, g->scan_ws_floats, s));
+            ZG_TRY(launch_part_norm(g->o, HV, HV, std::max(1, d.norm_groups), M, L.part_norm, eps, single ? &cv : nullptr, d_slot, s));
+            lin = Linear();
+            lin.A = g->o; lin.lda = HV; lin.B = L.o; lin.ldb = HV; lin.C = g->y; lin.ldc = W; lin.M = M; lin.N = W; lin.K = HV;
+            ZG_TRY(launch_linear(lin, f32, s));
+        } else if (d.mixer == ZG_LM_MIX_WINDOW_LINEAR) {
             const int G = d.kv_heads, HD = H * D, GD = G * D, GV = G * Vd, CC = HD + GD + GV, HV = H * Vd;
             const int HR = d.lin_heads, DR = d.lin_dim, VR = d.lin_vdim, HRD = HR * DR, HRV = HR * VR, NP = L.n_cat, OC = HV + HRV;
             const int og = CC, orq = CC + HV, org = orq + 2 * HRD + HRV;  // columns of the left gate, the right q | k | v, the right gate
@@ -848,12 +997,12 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
                                               s));
             }
             bool split = false;
-            ZG_TRY(launch_window_attention_split(g->ta, CC, g->o, OC, M, H, G, D, Vd, d.scale, d.window, d.keep_first, nullptr, nullptr, nullptr, d_pos,
+            ZG_TRY(launch_window_attention_split(g->ta, CC, g->o, OC, M, H, G, D, Vd, d.scale, KeyMask{d.window, d.keep_first, 0}, nullptr, nullptr, nullptr, d_pos,
                                                  d_slot, g->page_table, g->max_pages, g->P, ps.cache,
                                                  d.window > 0 ? d.window + d.keep_first : g->max_pages * g->P, g->win_ws, g->win_ws_floats, d_estart,
                                                  d_elen, n_ent, s, &split, g->proj + og, NP, d.left_scale));  // (the gate where the shares meet)
             if (!split) {
-                ZG_TRY(launch_window_attention(g->ta, CC, g->o, OC, M, H, G, D, Vd, d.scale, d.window, d.keep_first, nullptr, nullptr, nullptr, d_pos,
+                ZG_TRY(launch_window_attention(g->ta, CC, g->o, OC, M, H, G, D, Vd, d.scale, KeyMask{d.window, d.keep_first, 0}, nullptr, nullptr, nullptr, d_pos,
                                                d_slot, g->page_table, g->max_pages, g->P, ps.cache, s));
                 ZG_TRY(launch_norm_gate(g->o, OC, 1, HV, M, nullptr, eps, g->proj + og, NP, s, d.left_scale));
             }
@@ -874,11 +1023,11 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             // left: attention inside the window
             ZG_TRY(launch_window_prep(g->proj, NP, M, H, G, D, Vd, rot, L.vfreq, d_pos, d_slot, g->page_table, g->max_pages, g->P, ps.cache, s));
             bool split = false;
-            ZG_TRY(launch_window_attention_split(g->proj, NP, g->o, HV, M, H, G, D, Vd, d.scale, d.window, 0, L.sink, L.talk, L.vfreq, d_pos, d_slot,
+            ZG_TRY(launch_window_attention_split(g->proj, NP, g->o, HV, M, H, G, D, Vd, d.scale, KeyMask{d.window, 0, 0}, L.sink, L.talk, L.vfreq, d_pos, d_slot,
                                                  g->page_table, g->max_pages, g->P, ps.cache, d.window > 0 ? d.window : g->max_pages * g->P, g->win_ws,
                                                  g->win_ws_floats, d_estart, d_elen, n_ent, s, &split));
             if (!split)
-                ZG_TRY(launch_window_attention(g->proj, NP, g->o, HV, M, H, G, D, Vd, d.scale, d.window, 0, L.sink, L.talk, L.vfreq, d_pos, d_slot,
+                ZG_TRY(launch_window_attention(g->proj, NP, g->o, HV, M, H, G, D, Vd, d.scale, KeyMask{d.window, 0, 0}, L.sink, L.talk, L.vfreq, d_pos, d_slot,
                                                g->page_table, g->max_pages, g->P, ps.cache, s));
             lin = Linear();
             lin.A = g->o; lin.lda = HV; lin.B = L.o; lin.ldb = HV; lin.C = g->y; lin.ldc = W; lin.M = M; lin.N = W; lin.K = HV;
@@ -952,16 +1101,13 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             ZG_TRY(launch_linear(lin, f32, s));
             ZG_TRY(launch_head_norm_prep(g->proj, NP, M, H, G, D, eps, d.qtemp_coef, d.qtemp_every, d_pos, d_slot, g->page_table, g->max_pages, g->P,
                                          ps.cache, s));
-            // rows of the score workspace: as long as the longest sequence of this portion (a captured decode step replays at any
-            // length, so it takes the cache's capacity)
-            const int all_keys = g->max_pages * g->P;
-            const int key_cap = (single || capturing) ? (g->bucket_keys > 0 ? g->bucket_keys : all_keys) : std::min(all_keys, (g->step_keys + 63) / 64 * 64);
+            const int key_cap = whole_context_keys(single || capturing);
             bool split = false;
-            ZG_TRY(launch_window_attention_split(g->proj, NP, g->o, HD, M, H, G, D, D, d.scale, 0, 0, nullptr, nullptr, nullptr, d_pos, d_slot,
+            ZG_TRY(launch_window_attention_split(g->proj, NP, g->o, HD, M, H, G, D, D, d.scale, KeyMask(), nullptr, nullptr, nullptr, d_pos, d_slot,
                                                  g->page_table, g->max_pages, g->P, ps.cache, key_cap, g->win_ws, g->win_ws_floats, d_estart, d_elen,
                                                  n_ent, s, &split, nullptr, 0, 1.0f, shape));
             if (!split)
-                ZG_TRY(launch_window_attention(g->proj, NP, g->o, HD, M, H, G, D, D, d.scale, 0, 0, nullptr, nullptr, nullptr, d_pos, d_slot,
+                ZG_TRY(launch_window_attention(g->proj, NP, g->o, HD, M, H, G, D, D, d.scale, KeyMask(), nullptr, nullptr, nullptr, d_pos, d_slot,
                                                g->page_table, g->max_pages, g->P, ps.cache, s, shape));
             lin = Linear();
             lin.A = g->o; lin.lda = HD; lin.B = L.o; lin.ldb = HD; lin.C = g->y; lin.ldc = W; lin.M = M; lin.N = W; lin.K = HD;
@@ -978,28 +1124,37 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             lin.A = g->o; lin.lda = HV; lin.B = L.o; lin.ldb = HV; lin.C = g->y; lin.ldc = W; lin.M = M; lin.N = W; lin.K = HV;
             ZG_TRY(launch_linear(lin, f32, s));
         } else {
-            const int R = d.rot_dim, KR = d.kv_rank, QR = d.q_rank, HV = H * Vd, NP = QR + KR + R;
-            const Rotary rot{L.rot_freq, d.rot_dims, L.rot_amp};
+            const int R = d.rot_dim, KR = d.kv_rank, QR = d.q_rank, HV = H * Vd, LD = L.ld_cat;
+            const bool direct = QR == 0;  // queries projected directly (they sit in the fused projection's rows)
+            const Rotary rot{L.rot_freq, d.rot_dims, L.rot_amp, d.rot_halves};
             lin = Linear();
-            lin.A = hin; lin.lda = W; lin.B = L.dqkv; lin.ldb = W; lin.C = g->proj; lin.ldc = NP; lin.M = M; lin.N = NP; lin.K = W;
+            lin.A = hin; lin.lda = W; lin.B = L.dqkv; lin.ldb = W; lin.C = g->proj; lin.ldc = LD; lin.M = M; lin.N = L.n_cat; lin.K = W;
             ZG_TRY(launch_linear(lin, f32, s));
-            ZG_TRY(launch_latent_prep(g->proj, NP, M, QR, KR, R, L.dq_norm, L.dkv_norm, eps, rot, d_pos, d_slot, g->page_table, g->max_pages, g->P,
-                                      g->cq, ps.cache, s));
-            lin = Linear();
-            lin.A = g->cq; lin.lda = QR; lin.B = L.uq; lin.ldb = QR; lin.C = g->q; lin.ldc = H * (D + R); lin.M = M; lin.N = H * (D + R); lin.K = QR;
-            ZG_TRY(launch_linear(lin, f32, s));
+            const float* gate = d.head_gate ? g->proj + L.n_cat - H : nullptr;
+            const float* q = direct ? g->proj : g->q;
+            const int ldq = direct ? LD : H * (D + R);
+            if (direct) {
+                ZG_TRY(launch_latent_direct_prep(g->proj, LD, M, H, D, R, KR, H * (D + R), L.dkv_norm, eps, rot, d_pos, d_slot, g->page_table, g->max_pages,
+                                                 g->P, g->qa, d.kv_from > 0 ? nullptr : ps.cache, s));
+            } else {
+                ZG_TRY(launch_latent_prep(g->proj, LD, M, QR, KR, R, L.dq_norm, L.dkv_norm, eps, rot, d_pos, d_slot, g->page_table, g->max_pages, g->P,
+                                          g->cq, ps.cache, s));
+                lin = Linear();
+                lin.A = g->cq; lin.lda = QR; lin.B = L.uq; lin.ldb = QR; lin.C = g->q; lin.ldc = H * (D + R); lin.M = M; lin.N = H * (D + R); lin.K = QR;
+                ZG_TRY(launch_linear(lin, f32, s));
+            }
             lin = Linear();  // the unrotated query part carried into the latent space, head by head
-            lin.A = g->q; lin.lda = H * (D + R); lin.a_zoff = D + R; lin.B = L.ukT; lin.ldb = D; lin.b_zoff = (long long)KR * D;
+            lin.A = q; lin.lda = ldq; lin.a_zoff = D + R; lin.B = L.ukT; lin.ldb = D; lin.b_zoff = (long long)KR * D;
             lin.C = g->qa; lin.ldc = H * (KR + R); lin.c_zoff = KR + R; lin.M = M; lin.N = KR; lin.K = D; lin.nz = H;
             ZG_TRY(launch_linear(lin, f32, s));
-            ZG_TRY(launch_q_rotary(g->q, H * (D + R), g->qa, H * (KR + R), M, H, D, R, KR, rot, d_pos, s));
+            if (!direct) ZG_TRY(launch_q_rotary(g->q, H * (D + R), g->qa, H * (KR + R), M, H, D, R, KR, rot, d_pos, s));
             bool tiled = false;
             if (!f32 && !few)
                 ZG_TRY(launch_latent_attention_tiles(g->qa, g->ctx, M, H, KR, R, d.scale, d_estart, d_elen, d_eslot, n_ent, d_pos, g->page_table,
-                                                     g->max_pages, g->P, ps.cache, s, &tiled));
+                                                     g->max_pages, g->P, ps.cache, s, &tiled, gate, LD));
             if (!tiled)
                 ZG_TRY(launch_latent_attention(g->qa, g->ctx, M, H, KR, R, d.scale, d_pos, d_slot, g->page_table, g->max_pages, g->P, ps.cache,
-                                               g->attn_ws, g->attn_ws_floats, s));
+                                               g->attn_ws, g->attn_ws_floats, s, gate, LD));
             lin = Linear();  // values of the weighted latent, head by head
             lin.A = g->ctx; lin.lda = H * KR; lin.a_zoff = KR; lin.B = L.uv; lin.ldb = KR; lin.b_zoff = (long long)Vd * KR;
             lin.C = g->o; lin.ldc = HV; lin.c_zoff = Vd; lin.M = M; lin.N = Vd; lin.K = KR; lin.nz = H;
@@ -1023,12 +1178,7 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             const int F = d.ff_width;
             part = SumParts();
             if (d.ff == ZG_LM_FF_DENSE) {
-                lin = Linear();
-                lin.A = g->h; lin.lda = W; lin.B = L.up; lin.ldb = W; lin.C = g->u; lin.ldc = F; lin.M = M; lin.N = F; lin.K = W; lin.act = ACT_RELU2;
-                ZG_TRY(launch_linear(lin, f32, s));
-                lin = Linear();
-                lin.A = g->u; lin.lda = F; lin.B = L.down; lin.ldb = F; lin.C = g->y; lin.ldc = W; lin.M = M; lin.N = W; lin.K = F;
-                ZG_TRY(launch_linear(lin, f32, s));
+                ZG_TRY(dense_ff(L, g->h, g->y));
                 part.a = g->y;
             } else if (d.ff == ZG_LM_FF_MOE) {
                 const int E = d.experts, top = d.top, NA = M * top;
@@ -1102,12 +1252,7 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             const int F = d.ff_width;
             const float* fin = g->hc;
             if (d.ff == ZG_LM_FF_DENSE) {
-                lin = Linear();
-                lin.A = fin; lin.lda = W; lin.B = L.up; lin.ldb = W; lin.C = g->u; lin.ldc = F; lin.M = M; lin.N = F; lin.K = W; lin.act = ACT_RELU2;
-                ZG_TRY(launch_linear(lin, f32, s));
-                lin = Linear();
-                lin.A = g->u; lin.lda = F; lin.B = L.down; lin.ldb = F; lin.C = g->y2; lin.ldc = W; lin.M = M; lin.N = W; lin.K = F;
-                ZG_TRY(launch_linear(lin, f32, s));
+                ZG_TRY(dense_ff(L, fin, g->y2));
             } else if (d.ff == ZG_LM_FF_MOE) {
                 const int E = d.experts, top = d.top, NA = M * top;
                 const int UF = d.ff_act == ZG_LM_ACT_GELU ? F : 2 * F;
@@ -1194,12 +1339,7 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             hin = g->hc;
         }
         if (d.ff == ZG_LM_FF_DENSE) {
-            lin = Linear();
-            lin.A = hin; lin.lda = W; lin.B = L.up; lin.ldb = W; lin.C = g->u; lin.ldc = F; lin.M = M; lin.N = F; lin.K = W; lin.act = ACT_RELU2;
-            ZG_TRY(launch_linear(lin, f32, s));
-            lin = Linear();
-            lin.A = g->u; lin.lda = F; lin.B = L.down; lin.ldb = F; lin.C = g->y; lin.ldc = W; lin.M = M; lin.N = W; lin.K = F;
-            ZG_TRY(launch_linear(lin, f32, s));
+            ZG_TRY(dense_ff(L, hin, g->y));
             ZG_TRY(tail(g->y, nullptr, nullptr, 0, L.norm2b));
             if (!h_ready) ZG_TRY(launch_norm_add(g->x, g->y, L.norm2b, eps, M, W, s));
         } else if (d.ff == ZG_LM_FF_MOE) {
@@ -1235,7 +1375,7 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
         ZG_TRY(copy_trace(p));
     }
     // the rows the last tokens of the entries left for the token shift of their successors
-    if (!canon && !side && !tnorm) ZG_TRY(launch_commit_rows(g->shift_state, (size_t)g->n_passes * W, g->last_h, W, d_eslot, n_ent, W, g->n_passes, W, (size_t)NS * W, s));
+    if (!canon && !side && !tnorm && !g->no_shift) ZG_TRY(launch_commit_rows(g->shift_state, (size_t)g->n_passes * W, g->last_h, W, d_eslot, n_ent, W, g->n_passes, W, (size_t)NS * W, s));
 
     return ZG_OK;
 }
@@ -1478,6 +1618,7 @@ int zg_lm_create(zg_lm** out, const zg_lm_config* config, int device) {
     g->canon = config->canon_taps;
     g->side = (config->flags & ZG_LM_SIDE_BY_SIDE) != 0;
     g->tanh_norms = (config->flags & ZG_LM_TANH_NORMS) != 0;
+    g->no_shift = (config->flags & ZG_LM_NO_SHIFT) != 0;
     g->res_mult = config->residual_mult != 0.0f ? config->residual_mult : 1.0f;
     g->embed_scale = config->embed_scale != 0.0f ? config->embed_scale : 1.0f;
     int status = ZG_OK;
@@ -1510,6 +1651,20 @@ int zg_lm_create(zg_lm** out, const zg_lm_config* config, int device) {
                 status = ZG_ERR_ARG;
             }
         }
+    }
+    for (size_t i = 0; i < config->n_layers && status == ZG_OK; ++i) {  // a layer that reads another layer's latents
+        const zg_lm_layer& d = g->layers[i].d;
+        if (d.mixer != ZG_LM_MIX_LATENT_ATTENTION || d.kv_from <= 0) continue;
+        const size_t j = (size_t)d.kv_from - 1;
+        if (j >= i || g->layers[j].d.mixer != ZG_LM_MIX_LATENT_ATTENTION || g->layers[j].d.kv_from > 0 || g->layers[j].d.weights_of > 0 ||
+            d.weights_of > 0 || g->layers[j].d.kv_rank != d.kv_rank || g->layers[j].d.rot_dim != d.rot_dim) {
+            set_error("lm_create: layer %zu reads the latents of layer %zu, which must lie in front of it with latents of its own of the same sizes", i, j);
+            status = ZG_ERR_ARG;
+        }
+    }
+    if (status == ZG_OK && g->no_shift && (g->side || g->tanh_norms || g->canon != 0)) {
+        set_error("lm_create: a mixer that reads the norm as it is stands in sequential sublayers with RMS norms, without input convolution");
+        status = ZG_ERR_ARG;
     }
     if (status == ZG_OK && g->tanh_norms && (g->side || g->canon != 0 || (config->flags & ZG_LM_LOOP_READD))) {
         set_error("lm_create: the norms without statistics stand in sequential sublayers, without input convolution or re-added embedding");
@@ -1559,6 +1714,11 @@ int zg_lm_create(zg_lm** out, const zg_lm_config* config, int device) {
         const zg_lm_layer& d = g->layers[ps.layer].d;
         if (d.mixer == ZG_LM_MIX_LATENT_ATTENTION || d.mixer == ZG_LM_MIX_ATTENTION || (d.mixer == ZG_LM_MIX_PARALLEL && d.window == 0))
             attends = true, bounded = false;
+        if (d.mixer == ZG_LM_MIX_ROTARY_ATTENTION) {
+            attends = true;
+            if (d.chunk > 0 || d.window > 0) g->keep_tokens = std::max(g->keep_tokens, std::max(d.chunk, d.window));
+            else bounded = false, g->whole_context = true;
+        }
         if (d.mixer == ZG_LM_MIX_ATTENTION) g->whole_context = true;
         if (d.mixer == ZG_LM_MIX_PARALLEL && d.window > 0) {
             attends = true;
@@ -1633,7 +1793,7 @@ int zg_lm_create(zg_lm** out, const zg_lm_config* config, int device) {
             ZG_LM_TRY_HIP(hipMemcpy(L.slopes, sl.data(), sl.size() * sizeof(float), hipMemcpyHostToDevice));
         }
     for (LayerW& L : g->layers)
-        if ((L.d.mixer == ZG_LM_MIX_LATENT_ATTENTION || L.d.mixer == ZG_LM_MIX_PARALLEL) && L.d.weights_of == 0) {
+        if ((L.d.mixer == ZG_LM_MIX_LATENT_ATTENTION || L.d.mixer == ZG_LM_MIX_PARALLEL || L.d.mixer == ZG_LM_MIX_ROTARY_ATTENTION) && L.d.weights_of == 0) {
             std::vector<float> freq;
             rotary_table(L.d, freq, L.rot_amp);
             ZG_LM_TRY_HIP(hipMemcpy(L.rot_freq, freq.data(), std::max<size_t>(1, L.d.rot_dims / 2) * sizeof(float), hipMemcpyHostToDevice));

@@ -138,32 +138,10 @@ int launch_hgrn2_scan(const float* proj, int ld, float* out, int ldo, float* sta
                       const int* ent_len, const int* ent_slot, int n_entries, int M, int H, int D, int V, const float* bias, const float* low,
                       float* ws, size_t ws_floats, hipStream_t s, const float* decay = nullptr, const GlaGate* gla = nullptr);
 
-// ------------------------------------------------------------------------------------------------ latent attention
-// Rotary table of one layer: freq[i] for the rot_dims / 2 pairs (YaRN blend applied on the host) and the amplitude factor.
-// proj rows: [dq (q_rank) | dkv latent (KR) | rotated key part (R)].  Writes cq[m] = norm(dq) * wq, and the token's cache row
-// (latent = norm(dkv latent) * wkv | rotary(key part)) at its position: cache row of (slot, pos) = page_table[slot][pos / P] * P + pos % P.
-struct Rotary {
-    const float* freq;  // [dims / 2]
-    int dims;           // rotated dimensions (the first `dims` of the part; the rest pass)
-    float amp;
-};
-int launch_latent_prep(const float* proj, int ld, int M, int q_rank, int KR, int R, const float* wq, const float* wkv, float eps, Rotary rot,
-                       const int* row_pos, const int* row_slot, const int* page_table, int max_pages, int page_tokens, float* cq,
-                       float* cache, hipStream_t s);
-// qa[m][h][KR ..] = rotary(q[m][h][D ..]) — the rotated query part moved behind the absorbed part (which a batched Linear wrote).
-int launch_q_rotary(const float* q, int ldq, float* qa, int ldqa, int M, int H, int D, int R, int KR, Rotary rot, const int* row_pos, hipStream_t s);
-// ctx[m][h][:KR] = sum_j softmax_j( scale * qa[m][h] . cacherow(j) ) latent(j) over the keys j <= row_pos[m] of the row's sequence.
-// ws: fp32 workspace for the partials of split key ranges (steps of at most kGemvMaxRows rows: M * H * kAttnSplits * (KR + 2)
-// floats; without it whole key rows per workgroup).
-constexpr int kAttnSplits = 16;
-int launch_latent_attention(const float* qa, float* ctx, int M, int H, int KR, int R, float scale, const int* row_pos, const int* row_slot,
-                            const int* page_table, int max_pages, int page_tokens, const float* cache, float* ws, size_t ws_floats, hipStream_t s);
-
-// The same for prompt portions on the matrix cores (bf16 operands, fp32 scores / softmax / accumulation): 32 queries of one entry
-// and four heads per workgroup.  *taken = false when the latent is larger than the kernel's tiles hold (nothing launched).
-int launch_latent_attention_tiles(const float* qa, float* ctx, int M, int H, int KR, int R, float scale, const int* ent_start, const int* ent_len,
-                                  const int* ent_slot, int n_entries, const int* row_pos, const int* page_table, int max_pages, int page_tokens,
-                                  const float* cache, hipStream_t s, bool* taken);
+// The carry of a chunked recurrence: wsB [chunk][H][D][V] holds every chunk's end state from zero and receives its true start state,
+// wsA [chunk][H][a_rows] the chunk's decay (a_rows D: per row of the state, 1: per head); the slot's state moves on.
+int launch_state_carry(float* state, size_t slot_stride, const int* ent_len, const int* ent_slot, int n_entries, int H, int D, int V, float* wsB,
+                       const float* wsA, int a_rows, int chunk, hipStream_t s);
 
 // ------------------------------------------------------------------------------------------------ causal convolutions with a tail
 // out[m][c] = act( bias[c] + sum_j w[c][j] * in(m - (taps - 1) + j)[c]  (+ in(m)[c] with CONV_RESIDUAL) ),  in(.) = in[.] + pre_bias;
@@ -186,6 +164,73 @@ struct ConvArgs {
 // one_row_each: every entry brings exactly one row (decode steps): the convolution's own threads move the tails on, no second launch.
 int launch_causal_conv(const ConvArgs& a, int M, int n_entries, bool one_row_each, const int* row_off, const int* row_slot, const int* ent_start,
                        const int* ent_len, const int* ent_slot, hipStream_t s);
+
+// ------------------------------------------------------------------------------------------------ selective state space (Mamba-2)
+// Per entry and head h (B, C of group h / (H / G)), token by token on S = state[slot][h] ([N][V] fp32):
+//   dt = softplus(dt_raw + dt_bias[h]);  S <- exp(-exp(a_log[h]) dt) S + dt B x^T;  out = (S^T C + skip[h] x) * silu(z)
+// xbc rows [x (H V) | B (G N) | C (G N)]: convolved and activated — or, with conv != null (steps of one row per entry), the raw
+// projection columns: the kernel applies the convolution (bias, silu) over the slot's tail itself and leaves the tail alone.
+struct SsdArgs {
+    const float* xbc = nullptr;
+    int ld_xbc = 0;
+    const float* dt = nullptr;   // raw step sizes [H]
+    const float* z = nullptr;    // gates [H V]
+    int ld_proj = 0;             // row stride of dt and z
+    const float *dt_bias = nullptr, *a_log = nullptr, *skip = nullptr;
+    int H = 0, G = 1, N = 0, V = 0;
+    float* out = nullptr;
+    int ldo = 0;
+    float* state = nullptr;
+    size_t slot_stride = 0;
+};
+constexpr int kSsdMaxState = 256;
+// ws: workspace of the chunk-parallel form, ssd_workspace(M, n_entries, ...) floats (null or too small: token by token)
+size_t ssd_workspace(int M, int n_entries, int H, int N, int V);
+int launch_ssd_scan(const SsdArgs& a, const ConvArgs* conv, int M, const int* ent_start, const int* ent_len, const int* ent_slot, int n_entries,
+                    float* ws, size_t ws_floats, hipStream_t s);
+// In place: v[m] cut into `parts` equal parts, each divided by its own root mean square, times w (one weight per channel).
+// conv != null (steps of one row per entry): conv's tail is moved on by the row's inputs in the same launch.
+int launch_part_norm(float* v, int ld, int width, int parts, int M, const float* w, float eps, const ConvArgs* conv, const int* row_slot, hipStream_t s);
+// In place over M rows of F floats: a N(z) + b N(z^2) + c N(z^3) + e with N over the row; act holds a, b, c, e.
+int launch_polynorm(float* z, int ld, int F, int M, const float* act, float eps, hipStream_t s);
+
+// ------------------------------------------------------------------------------------------------ latent attention
+// Rotary table of one layer: freq[i] for the rot_dims / 2 pairs (YaRN blend applied on the host) and the amplitude factor.
+// proj rows: [dq (q_rank) | dkv latent (KR) | rotated key part (R)].  Writes cq[m] = norm(dq) * wq, and the token's cache row
+// (latent = norm(dkv latent) * wkv | rotary(key part)) at its position: cache row of (slot, pos) = page_table[slot][pos / P] * P + pos % P.
+struct Rotary {
+    const float* freq;  // [dims / 2]
+    int dims;           // rotated dimensions (the first `dims` of the part; the rest pass)
+    float amp;
+    int halves = 0;     // 0: pairs (2i, 2i + 1); 1: pairs (i, i + dims / 2)
+};
+int launch_latent_prep(const float* proj, int ld, int M, int q_rank, int KR, int R, const float* wq, const float* wkv, float eps, Rotary rot,
+                       const int* row_pos, const int* row_slot, const int* page_table, int max_pages, int page_tokens, float* cq,
+                       float* cache, hipStream_t s);
+// Queries projected directly: proj rows [q (H (D + R)) | dkv latent (KR) | rotated key part (R) at column kv_col].  qa[m][h][KR ..] =
+// rotary(q[m][h][D ..]) and, with cache != null, the token's cache row as above — one launch.  cache == null: the layer reads another
+// layer's latents (no dkv columns).
+int launch_latent_direct_prep(const float* proj, int ld, int M, int H, int D, int R, int KR, int kv_col, const float* wkv, float eps, Rotary rot,
+                              const int* row_pos, const int* row_slot, const int* page_table, int max_pages, int page_tokens, float* qa, float* cache,
+                              hipStream_t s);
+// qa[m][h][KR ..] = rotary(q[m][h][D ..]) — the rotated query part moved behind the absorbed part (which a batched Linear wrote).
+int launch_q_rotary(const float* q, int ldq, float* qa, int ldqa, int M, int H, int D, int R, int KR, Rotary rot, const int* row_pos, hipStream_t s);
+// ctx[m][h][:KR] = sum_j softmax_j( scale * qa[m][h] . cacherow(j) ) latent(j) over the keys j <= row_pos[m] of the row's sequence.
+// ws: fp32 workspace for the partials of split key ranges (steps of at most kGemvMaxRows rows: M * H * kAttnSplits * (KR + 2)
+// floats; without it whole key rows per workgroup).
+// gate != null: head h's result is multiplied by sigmoid(gate[m ldg + h]).
+constexpr int kAttnSplits = 16;
+int launch_latent_attention(const float* qa, float* ctx, int M, int H, int KR, int R, float scale, const int* row_pos, const int* row_slot,
+                            const int* page_table, int max_pages, int page_tokens, const float* cache, float* ws, size_t ws_floats, hipStream_t s,
+                            const float* gate = nullptr, int ldg = 0);
+
+// The same for prompt portions on the matrix cores (bf16 operands, fp32 scores / softmax / accumulation): 32 queries of one entry
+// and four heads per workgroup.  *taken = false when the latent is larger than the kernel's tiles hold (nothing launched).
+int launch_latent_attention_tiles(const float* qa, float* ctx, int M, int H, int KR, int R, float scale, const int* ent_start, const int* ent_len,
+                                  const int* ent_slot, int n_entries, const int* row_pos, const int* page_table, int max_pages, int page_tokens,
+                                  const float* cache, hipStream_t s, bool* taken, const float* gate = nullptr, int ldg = 0);
+
+// ------------------------------------------------------------------------------------------------ input convolution of decode rows, residual sum
 // Steps of one row per entry: [x += x0] or [x += norm(y) * (1 + wb), y = yl or the mean of the two normed branches yl, yr with
 // plain weights wl, wr], then h = norm(x) * (1 + wn), out = h + conv(h) over the slot's tail, the tail moved on — one launch.
 // *taken = false for rows too wide for its registers (nothing launched).
@@ -199,11 +244,13 @@ int launch_add_rows(float* x, const float* y, int M, int W, hipStream_t s);
 // proj rows [q (H D) | k (G D) | v (G V)]: q rotated in place; the rotated key and the value rotated over all V channels (pair i by
 // pos * vfreq[i]) written to the token's cache row [G D | G V]; the page of (slot, pos) is page_table[slot][(pos / P) % max_pages]:
 // a ring, so that a sequence whose old pages have been given back can grow beyond max_pages * P positions.
+// vfreq == null: the values are cached as they are.
 int launch_window_prep(float* proj, int ld, int M, int H, int G, int D, int V, Rotary rot, const float* vfreq, const int* row_pos,
                        const int* row_slot, const int* page_table, int max_pages, int page_tokens, float* cache, hipStream_t s);
 // out[m][h] = turn_back_pos( sum_j w_h(j) value_(h / (H/G))(j) ),  w_h = sum_g talk[h][g] p_g,
 // p_g(j) = exp(s_g(j)) / (exp(sink_g) + sum_j' exp(s_g(j'))),  s_g(j) = scale q_g . k(j),  over the keys pos - window < j <= pos
-// (window 0: all j <= pos).  sink / talk may be null (no sink / no mix).
+// (window 0: all j <= pos; chunk > 0: the keys of pos's own chunk [n chunk, (n + 1) chunk) up to pos).  sink / talk may be null (no
+// sink / no mix).
 // keep_first > 0: beyond the window the first keep_first positions of the sequence stay visible (a row's keys are then numbered
 // kept tokens first, then the window).  vfreq == null: values are cached unrotated and nothing is turned back.
 // shape: what becomes of a scaled score before the softmax — capped (cap > 0: cap tanh(s / cap)), then less slope[h] per position
@@ -212,8 +259,12 @@ struct ScoreShape {
     float cap = 0.0f;
     const float* slope = nullptr;  // [H]
 };
-int launch_window_attention(const float* q, int ldq, float* out, int ldo, int M, int H, int G, int D, int V, float scale, int window,
-                            int keep_first, const float* sink, const float* talk, const float* vfreq, const int* row_pos, const int* row_slot,
+// which keys at or before a query it sees: a sliding window (with the sequence's first keep tokens behind it), its chunk, or all
+struct KeyMask {
+    int window = 0, keep = 0, chunk = 0;
+};
+int launch_window_attention(const float* q, int ldq, float* out, int ldo, int M, int H, int G, int D, int V, float scale, KeyMask mask,
+                            const float* sink, const float* talk, const float* vfreq, const int* row_pos, const int* row_slot,
                             const int* page_table, int max_pages, int page_tokens, const float* cache, hipStream_t s,
                             ScoreShape shape = ScoreShape());
 // The prep of attention whose q and k are divided by their root mean square PER HEAD (no weight) and whose values are the
@@ -239,8 +290,8 @@ int launch_whole_norm_prep(float* qkv, int ld, int M, int HD, int GD, int GV, co
 // rows with consecutive positions: ent_start / ent_len).
 constexpr int kWinSplits = 64;
 size_t window_split_workspace(int rows, int H, int V, int key_capacity, int* n_split_out);
-int launch_window_attention_split(const float* q, int ldq, float* out, int ldo, int M, int H, int G, int D, int V, float scale, int window,
-                                  int keep_first, const float* sink, const float* talk, const float* vfreq, const int* row_pos, const int* row_slot,
+int launch_window_attention_split(const float* q, int ldq, float* out, int ldo, int M, int H, int G, int D, int V, float scale, KeyMask mask,
+                                  const float* sink, const float* talk, const float* vfreq, const int* row_pos, const int* row_slot,
                                   const int* page_table, int max_pages, int page_tokens, const float* cache, int key_capacity, float* ws,
                                   size_t ws_floats, const int* ent_start, const int* ent_len, int n_entries, hipStream_t s, bool* taken,
                                   const float* out_gate = nullptr, int ld_gate = 0, float out_factor = 1.0f, ScoreShape shape = ScoreShape());

@@ -566,14 +566,14 @@ __global__ __launch_bounds__(256) void hgrn2_scan_kernel(const float* proj, int 
 
 // phase B: one thread per state element walks the chunks of its entry
 __global__ __launch_bounds__(256) void hgrn2_carry_kernel(float* state, size_t slot_stride, const int* ent_len, const int* ent_slot, int n_entries, int H,
-                                                          int D, int V, float* wsB, const float* wsA, int chunk) {
+                                                          int D, int V, float* wsB, const float* wsA, int a_rows, int chunk) {
     const int e = blockIdx.y;
     const size_t n = (size_t)H * D * V, idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= n) return;
     int first = 0;
     for (int k = 0; k < e; ++k) first += (ent_len[k] + chunk - 1) / chunk;
     const int nc = (ent_len[e] + chunk - 1) / chunk;
-    const size_t hi = idx / V;  // (head, row)
+    const size_t ai = idx / ((size_t)V * (D / a_rows)), na = (size_t)H * a_rows;  // the decay of the element's (head, row), or of its head
     float* slot = state + (size_t)ent_slot[e] * slot_stride;
     float S = slot[idx];
     for (int c0 = 0; c0 < nc; c0 += 8) {  // eight chunks' operands requested together: the chain itself is eight multiply-adds
@@ -582,7 +582,7 @@ __global__ __launch_bounds__(256) void hgrn2_carry_kernel(float* state, size_t s
         for (int u = 0; u < 8; ++u) {
             const int c = min(c0 + u, nc - 1);
             Bv[u] = wsB[(size_t)(first + c) * n + idx];
-            Av[u] = wsA[(size_t)(first + c) * H * D + hi];
+            Av[u] = wsA[(size_t)(first + c) * na + ai];
         }
 #pragma unroll
         for (int u = 0; u < 8; ++u)
@@ -750,13 +750,14 @@ __device__ __forceinline__ size_t cache_row(const int* page_table, int max_pages
     return (size_t)page_table[(size_t)slot * max_pages + pos / page_tokens] * page_tokens + pos % page_tokens;
 }
 
-// the interleaved pair (2i, 2i + 1) of `src` at position pos, rotated by pos * freq[i]; angle and product in fp32
+// pair i of `src` (channels (2i, 2i + 1), or (i, i + dims / 2)) at position pos, rotated by pos * freq[i]; angle and product in fp32
 __device__ __forceinline__ void rotate_pair(const float* src, float* dst, int i, int pos, const Rotary& rot) {
     const float a = (float)pos * rot.freq[i];
     const float c = cosf(a) * rot.amp, s = sinf(a) * rot.amp;
-    const float u = src[2 * i], v = src[2 * i + 1];
-    dst[2 * i] = u * c - v * s;
-    dst[2 * i + 1] = v * c + u * s;
+    const int a0 = rot.halves ? i : 2 * i, a1 = rot.halves ? i + rot.dims / 2 : 2 * i + 1;
+    const float u = src[a0], v = src[a1];
+    dst[a0] = u * c - v * s;
+    dst[a1] = v * c + u * s;
 }
 
 __global__ __launch_bounds__(256) void latent_prep_kernel(const float* proj, int ld, int q_rank, int KR, int R, const float* wq, const float* wkv,
@@ -790,14 +791,45 @@ __global__ __launch_bounds__(256) void q_rotary_kernel(const float* q, int ldq, 
     }
 }
 
+// Queries projected directly: blockIdx.y == 0 rotates the heads' query parts into qa, blockIdx.y == 1 (layers with latents of their
+// own) norms the latent, rotates the shared key part and files both in the token's cache row.
+__global__ __launch_bounds__(256) void latent_direct_prep_kernel(const float* proj, int ld, int H, int D, int R, int KR, int kv_col, const float* wkv,
+                                                                 float eps, Rotary rot, const int* row_pos, const int* row_slot, const int* page_table,
+                                                                 int max_pages, int page_tokens, float* qa, float* cache) {
+    __shared__ float s_red[8];
+    const int m = blockIdx.x, pos = row_pos[m], half = rot.dims / 2;
+    const float* row = proj + (size_t)m * ld;
+    if (blockIdx.y == 0) {
+        const int rest = R - rot.dims, per = half + rest;
+        for (int idx = threadIdx.x; idx < H * per; idx += blockDim.x) {
+            const int h = idx / per, i = idx % per;
+            const float* src = row + (size_t)h * (D + R) + D;
+            float* dst = qa + ((size_t)m * H + h) * (KR + R) + KR;
+            if (i < half) rotate_pair(src, dst, i, pos, rot);
+            else dst[rot.dims + i - half] = src[rot.dims + i - half];
+        }
+        return;
+    }
+    const float* lat = row + kv_col;
+    const float rc = row_inv_rms(lat, KR, eps, s_red);
+    float* crow = cache + cache_row(page_table, max_pages, page_tokens, row_slot[m], pos) * (size_t)(KR + R);
+    for (int i = threadIdx.x; i < KR; i += blockDim.x) crow[i] = lat[i] * rc * wkv[i];
+    const float* kr = lat + KR;
+    for (int i = threadIdx.x; i < half; i += blockDim.x) rotate_pair(kr, crow + KR, i, pos, rot);
+    for (int i = rot.dims + threadIdx.x; i < R; i += blockDim.x) crow[KR + i] = kr[i];
+}
+
 // One workgroup per (row, head).  The lanes of a wave split the KR + R dimensions of a cache row (ND per lane); a wave walks
 // its share of the keys four at a time with a running (maximum, sum, weighted latent) and the four waves are merged at the end.
 // With n_split > 1 (decode steps: few rows, long key ranges) grid.z workgroups share a row's keys in ranges of at least 64
 // and leave (maximum, sum, weighted latent) partials in ws for latent_merge_kernel.
+// gate (may be null): head h's result is multiplied by sigmoid(gate[m ldg + h]) where it is written.
+__device__ __forceinline__ float head_gate_f(const float* gate, int ldg, size_t m, int h) { return gate ? sigmoid_f(gate[m * ldg + h]) : 1.0f; }
+
 template <int ND>
 __global__ __launch_bounds__(256) void latent_attention_kernel(const float* qa, float* ctx, int H, int KR, int R, float scale, const int* row_pos,
                                                                const int* row_slot, const int* page_table, int max_pages, int page_tokens,
-                                                               const float* cache, float* ws, int n_split) {
+                                                               const float* cache, float* ws, int n_split, const float* gate, int ldg) {
     __shared__ float s_m[4], s_l[4];
     __shared__ float s_acc[4][ND * 64];
     const int m = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -883,11 +915,12 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const float* qa, 
         return;
     }
     float* out = ctx + ((size_t)m * H + h) * KR;
+    const float gf = head_gate_f(gate, ldg, m, h);
     for (int d = threadIdx.x; d < KR; d += blockDim.x) {
         float a = 0.0f;
 #pragma unroll
         for (int w = 0; w < 4; ++w) a = fmaf(wgt[w], s_acc[w][d], a);
-        out[d] = a / L;
+        out[d] = a / L * gf;
     }
 }
 
@@ -905,7 +938,7 @@ template <int NKS, int NT>  // 16 NKS >= KR + R (score dimensions), 32 NT >= KR 
 __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(const float* qa, float* ctx, int H, int KR, int R, float scale,
                                                                     const int* ent_start, const int* ent_len, const int* ent_slot, int n_entries,
                                                                     const int* row_pos, const int* page_table, int max_pages, int page_tokens,
-                                                                    const float* cache) {
+                                                                    const float* cache, const float* gate, int ldg) {
     constexpr int DTp = NKS * 16, KS_LD = DTp + 8, VT_LD = 40;
     __shared__ __attribute__((aligned(16))) bf16_t Ks[32 * KS_LD];
     __shared__ __attribute__((aligned(16))) bf16_t Vt[NT * 32 * VT_LD];
@@ -1059,18 +1092,20 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(const float*
     const float L = lsum + __shfl_xor(lsum, 32, 64);
     if (!q_ok) return;
     float* out = ctx + ((size_t)(m_first + r) * H + h) * KR;
+    const float gf = head_gate_f(gate, ldg, (size_t)(m_first + r), h);
 #pragma unroll
     for (int t = 0; t < NT; ++t)
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
             const int d = t * 32 + 8 * (i >> 2) + 4 * hf + (i & 3);
-            if (d < KR) out[d] = o[t][i] / L;
+            if (d < KR) out[d] = o[t][i] / L * gf;
         }
 }
 
 // ctx[m][h] from the partials of latent_attention_kernel, in a fixed order (the result does not depend on timing); only the
 // ranges that held keys are read
-__global__ __launch_bounds__(256) void latent_merge_kernel(const float* ws, float* ctx, int H, int KR, int n_split, const int* row_pos) {
+__global__ __launch_bounds__(256) void latent_merge_kernel(const float* ws, float* ctx, int H, int KR, int n_split, const int* row_pos, const float* gate,
+                                                           int ldg) {
     __shared__ float s_w[64];
     __shared__ float s_L;
     const int m = blockIdx.x, h = blockIdx.y, n_keys = row_pos[m] + 1;
@@ -1089,11 +1124,11 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const float* ws, floa
     }
     __syncthreads();
     float* out = ctx + ((size_t)m * H + h) * KR;
-    const float L = s_L;
+    const float L = s_L, gf = head_gate_f(gate, ldg, m, h);
     for (int d = threadIdx.x; d < KR; d += blockDim.x) {
         float a = 0.0f;
         for (int sidx = 0; sidx < used; ++sidx) a = fmaf(s_w[sidx], part[(size_t)sidx * (KR + 2) + 2 + d], a);
-        out[d] = a / L;
+        out[d] = a / L * gf;
     }
 }
 
@@ -1261,6 +1296,17 @@ int launch_norm_plain(float* v, int ld, int rows_per_m, int width, int M, const 
     return ZG_OK;
 }
 
+int launch_state_carry(float* state, size_t slot_stride, const int* ent_len, const int* ent_slot, int n_entries, int H, int D, int V, float* wsB,
+                       const float* wsA, int a_rows, int chunk, hipStream_t s) {
+    const size_t n = (size_t)H * D * V;
+    if (n_entries <= 0 || n == 0) return ZG_OK;
+    ZG_REQUIRE(a_rows == 1 || a_rows == D, ZG_ERR_ARG, "state carry: %d decays per head of %d rows", a_rows, D);
+    hgrn2_carry_kernel<<<dim3((unsigned)((n + 255) / 256), n_entries), 256, 0, s>>>(state, slot_stride, ent_len, ent_slot, n_entries, H, D, V, wsB, wsA, a_rows,
+                                                                                  chunk);
+    ZG_HIP(hipGetLastError());
+    return ZG_OK;
+}
+
 int launch_hgrn2_scan(const float* proj, int ld, float* out, int ldo, float* state, size_t slot_stride, const int* ent_start,
                       const int* ent_len, const int* ent_slot, int n_entries, int M, int H, int D, int V, const float* bias, const float* low,
                       float* ws, size_t ws_floats, hipStream_t s, const float* decay, const GlaGate* gla) {
@@ -1279,9 +1325,7 @@ int launch_hgrn2_scan(const float* proj, int ld, float* out, int ldo, float* sta
             const int tiles = ((D + 31) / 32) * ((V + 31) / 32);
             linear_chunk_state_kernel<<<dim3(n_chunks, H, std::min(16, (tiles + 3) / 4)), 256, 0, s>>>(proj, ld, ent_start, ent_len, n_entries, H, D, V, decay, cB, cA);
             ZG_HIP(hipGetLastError());
-            hgrn2_carry_kernel<<<dim3((unsigned)((hf + 255) / 256), n_entries), 256, 0, s>>>(state, slot_stride, ent_len, ent_slot, n_entries, H, D, V, cB,
-                                                                                          cA, kLinChunk);
-            ZG_HIP(hipGetLastError());
+            ZG_TRY(launch_state_carry(state, slot_stride, ent_len, ent_slot, n_entries, H, D, V, cB, cA, D, kLinChunk, s));
             const int dh = (D + 1) / 2;
             if (dh <= 8) linear_chunk_out_kernel<8><<<grid, 256, 0, s>>>(proj, ld, out, ldo, ent_start, ent_len, n_entries, H, D, V, decay, cB);
             else if (dh <= 16) linear_chunk_out_kernel<16><<<grid, 256, 0, s>>>(proj, ld, out, ldo, ent_start, ent_len, n_entries, H, D, V, decay, cB);
@@ -1330,9 +1374,7 @@ int launch_hgrn2_scan(const float* proj, int ld, float* out, int ldo, float* sta
     }
     ZG_SCAN_G(max_chunks, SCAN_A);
     ZG_HIP(hipGetLastError());
-    hgrn2_carry_kernel<<<dim3((unsigned)((head_floats + 255) / 256), n_entries), 256, 0, s>>>(state, slot_stride, ent_len, ent_slot, n_entries, H, D, V,
-                                                                                                wsB, wsA, kScanChunk);
-    ZG_HIP(hipGetLastError());
+    ZG_TRY(launch_state_carry(state, slot_stride, ent_len, ent_slot, n_entries, H, D, V, wsB, wsA, D, kScanChunk, s));
     ZG_SCAN_G(max_chunks, SCAN_C);
     ZG_HIP(hipGetLastError());
 #undef ZG_SCAN_G
@@ -1352,6 +1394,17 @@ int launch_latent_prep(const float* proj, int ld, int M, int q_rank, int KR, int
     return ZG_OK;
 }
 
+int launch_latent_direct_prep(const float* proj, int ld, int M, int H, int D, int R, int KR, int kv_col, const float* wkv, float eps, Rotary rot,
+                              const int* row_pos, const int* row_slot, const int* page_table, int max_pages, int page_tokens, float* qa, float* cache,
+                              hipStream_t s) {
+    if (M <= 0) return ZG_OK;
+    ZG_REQUIRE(rot.dims % 2 == 0 && rot.dims <= R, ZG_ERR_ARG, "rotary: %d rotated dimensions of a part of %d", rot.dims, R);
+    latent_direct_prep_kernel<<<dim3(M, cache ? 2 : 1), 256, 0, s>>>(proj, ld, H, D, R, KR, kv_col, wkv, eps, rot, row_pos, row_slot, page_table, max_pages,
+                                                                     page_tokens, qa, cache);
+    ZG_HIP(hipGetLastError());
+    return ZG_OK;
+}
+
 int launch_q_rotary(const float* q, int ldq, float* qa, int ldqa, int M, int H, int D, int R, int KR, Rotary rot, const int* row_pos,
                     hipStream_t s) {
     if (M <= 0 || R <= 0) return ZG_OK;
@@ -1362,14 +1415,14 @@ int launch_q_rotary(const float* q, int ldq, float* qa, int ldqa, int M, int H, 
 
 int launch_latent_attention_tiles(const float* qa, float* ctx, int M, int H, int KR, int R, float scale, const int* ent_start, const int* ent_len,
                                   const int* ent_slot, int n_entries, const int* row_pos, const int* page_table, int max_pages, int page_tokens,
-                                  const float* cache, hipStream_t s, bool* taken) {
+                                  const float* cache, hipStream_t s, bool* taken, const float* gate, int ldg) {
     *taken = false;
     if (M <= 0 || n_entries <= 0) return ZG_OK;
     const int DT = KR + R;
     const dim3 grid((M + 31) / 32 + n_entries, (H + 3) / 4);
 #define ZG_ATT_T(NKS_, NT_)                                                                                                                      \
     latent_attention_mfma_kernel<NKS_, NT_><<<grid, 256, 0, s>>>(qa, ctx, H, KR, R, scale, ent_start, ent_len, ent_slot, n_entries, row_pos, page_table, \
-                                                                 max_pages, page_tokens, cache)
+                                                                 max_pages, page_tokens, cache, gate, ldg)
     if (DT <= 96 && KR <= 64) ZG_ATT_T(6, 2);
     else if (DT <= 160 && KR <= 128) ZG_ATT_T(10, 4);
     else if (DT <= 288 && KR <= 256) ZG_ATT_T(18, 8);
@@ -1383,7 +1436,7 @@ int launch_latent_attention_tiles(const float* qa, float* ctx, int M, int H, int
 
 int launch_latent_attention(const float* qa, float* ctx, int M, int H, int KR, int R, float scale, const int* row_pos, const int* row_slot,
                             const int* page_table, int max_pages, int page_tokens, const float* cache, float* ws, size_t ws_floats,
-                            hipStream_t s) {
+                            hipStream_t s, const float* gate, int ldg) {
     if (M <= 0) return ZG_OK;
     const int nd = (KR + R + 63) / 64;
     ZG_REQUIRE(nd <= 16, ZG_ERR_UNSUPPORTED, "latent attention: %d cached dimensions per token (at most 1024)", KR + R);
@@ -1394,7 +1447,7 @@ int launch_latent_attention(const float* qa, float* ctx, int M, int H, int KR, i
     const dim3 grid(M, H, n_split);
 #define ZG_ATT(ND_)                                                                                                                           \
     latent_attention_kernel<ND_><<<grid, 256, 0, s>>>(qa, ctx, H, KR, R, scale, row_pos, row_slot, page_table, max_pages, page_tokens, cache, ws, \
-                                                      n_split)
+                                                      n_split, gate, ldg)
     if (nd <= 1) ZG_ATT(1);
     else if (nd <= 2) ZG_ATT(2);
     else if (nd <= 3) ZG_ATT(3);
@@ -1406,7 +1459,7 @@ int launch_latent_attention(const float* qa, float* ctx, int M, int H, int KR, i
 #undef ZG_ATT
     ZG_HIP(hipGetLastError());
     if (n_split > 1) {
-        latent_merge_kernel<<<dim3(M, H), 256, 0, s>>>(ws, ctx, H, KR, n_split, row_pos);
+        latent_merge_kernel<<<dim3(M, H), 256, 0, s>>>(ws, ctx, H, KR, n_split, row_pos, gate, ldg);
         ZG_HIP(hipGetLastError());
     }
     return ZG_OK;

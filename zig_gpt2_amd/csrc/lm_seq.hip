@@ -195,8 +195,9 @@ __global__ __launch_bounds__(256) void norm_conv_single_kernel(float* x, const f
 }
 
 // ------------------------------------------------------------------------------------------------ windowed attention
-// proj rows: [q (H D) | k (G D) | v (G V)].  q is rotated in place (pairs (2i, 2i + 1) below rot.dims); the rotated key and the
-// value rotated over ALL its channels (pair i by pos * vfreq[i]) go to the token's cache row [G D | G V].
+// proj rows: [q (H D) | k (G D) | v (G V)].  q is rotated in place (pairs (2i, 2i + 1) below rot.dims, or (i, i + dims / 2)); the
+// rotated key and the value rotated over ALL its channels (pair i by pos * vfreq[i]; vfreq null: as it is) go to the token's cache
+// row [G D | G V].
 __global__ __launch_bounds__(256) void window_prep_kernel(float* proj, int ld, int H, int G, int D, int V, Rotary rot, const float* vfreq,
                                                           const int* row_pos, const int* row_slot, const int* page_table, int max_pages,
                                                           int page_tokens, float* cache) {
@@ -209,12 +210,13 @@ __global__ __launch_bounds__(256) void window_prep_kernel(float* proj, int ld, i
     const int half = rot.dims / 2;
     for (int idx = threadIdx.x; idx < H * half; idx += blockDim.x) {
         const int h = idx / half, i = idx % half;
-        float* p = row + (size_t)h * D + 2 * i;
+        float* p = row + (size_t)h * D + (rot.halves ? i : 2 * i);
+        const int step = rot.halves ? half : 1;
         float sn, cs;
         sincosf(fpos * rot.freq[i], &sn, &cs);
-        const float a = p[0], b = p[1];
+        const float a = p[0], b = p[step];
         p[0] = (a * cs - b * sn) * rot.amp;
-        p[1] = (b * cs + a * sn) * rot.amp;
+        p[step] = (b * cs + a * sn) * rot.amp;
     }
     const float* k = row + (size_t)H * D;
     for (int idx = threadIdx.x; idx < G * D; idx += blockDim.x) {
@@ -222,9 +224,10 @@ __global__ __launch_bounds__(256) void window_prep_kernel(float* proj, int ld, i
         float out;
         if (i < rot.dims) {
             float sn, cs;
-            sincosf(fpos * rot.freq[i >> 1], &sn, &cs);
-            const float own = k[idx], other = k[idx - i + (i ^ 1)];
-            out = ((i & 1) ? own * cs + other * sn : own * cs - other * sn) * rot.amp;
+            const bool second = rot.halves ? i >= half : (i & 1);
+            sincosf(fpos * rot.freq[rot.halves ? (second ? i - half : i) : i >> 1], &sn, &cs);
+            const float own = k[idx], other = k[idx - i + (rot.halves ? (second ? i - half : i + half) : i ^ 1)];
+            out = (second ? own * cs + other * sn : own * cs - other * sn) * rot.amp;
         } else {
             out = k[idx];
         }
@@ -233,6 +236,10 @@ __global__ __launch_bounds__(256) void window_prep_kernel(float* proj, int ld, i
     const float* v = k + (size_t)G * D;
     for (int idx = threadIdx.x; idx < G * V; idx += blockDim.x) {
         const int i = idx % V;
+        if (!vfreq) {
+            crow[(size_t)G * D + idx] = v[idx];
+            continue;
+        }
         float sn, cs;
         sincosf(fpos * vfreq[i >> 1], &sn, &cs);
         const float own = v[idx], other = v[idx - i + (i ^ 1)];
@@ -251,10 +258,10 @@ __global__ __launch_bounds__(256) void window_prep_kernel(float* proj, int ld, i
 struct KeySpan {
     int j_lo, n_first, n_keys;
 };
-__device__ __forceinline__ KeySpan key_span(int pos, int window, int keep) {
+__device__ __forceinline__ KeySpan key_span(int pos, const KeyMask& mask) {
     KeySpan k;
-    k.j_lo = window > 0 ? max(0, pos - window + 1) : 0;
-    k.n_first = min(keep, k.j_lo);
+    k.j_lo = mask.chunk > 0 ? pos - pos % mask.chunk : mask.window > 0 ? max(0, pos - mask.window + 1) : 0;
+    k.n_first = min(mask.keep, k.j_lo);
     k.n_keys = k.n_first + pos - k.j_lo + 1;
     return k;
 }
@@ -272,7 +279,7 @@ constexpr int kWinMaxHeads = 64;
 constexpr int kWinAcc = 16;  // outputs per thread: H * V <= 256 * kWinAcc
 
 __global__ __launch_bounds__(256) void window_attention_kernel(const float* q, int ldq, float* out, int ldo, int H, int G, int D, int V,
-                                                               float scale, int window, int keep, const float* sink, const float* talk,
+                                                               float scale, KeyMask mask, const float* sink, const float* talk,
                                                                const float* vfreq, const int* row_pos, const int* row_slot,
                                                                const int* page_table, int max_pages, int page_tokens, const float* cache,
                                                                const ScoreShape shape) {
@@ -287,7 +294,7 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const float* q, i
     const int m = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int pos = row_pos[m];
     const int* pages = page_table + (size_t)row_slot[m] * max_pages;
-    const KeySpan span = key_span(pos, window, keep);
+    const KeySpan span = key_span(pos, mask);
     const int n_keys = span.n_keys;
     const int rep = H / G;
     const size_t cstride = (size_t)G * (D + V);
@@ -394,8 +401,8 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const float* q, i
 // A share is ceil(keys of the row / splits) consecutive keys: the order of every sum depends on the position alone.
 constexpr int kMixTile = 32;
 
-__device__ __forceinline__ KeySpan window_range(int pos, int window, int keep, int n_split, int split, int& k0, int& k1) {
-    const KeySpan span = key_span(pos, window, keep);
+__device__ __forceinline__ KeySpan window_range(int pos, const KeyMask& mask, int n_split, int split, int& k0, int& k1) {
+    const KeySpan span = key_span(pos, mask);
     const int chunk = (span.n_keys + n_split - 1) / n_split;
     k0 = min(span.n_keys, split * chunk);
     k1 = min(span.n_keys, k0 + chunk);
@@ -406,8 +413,7 @@ constexpr int kScoreTile = 128;  // keys whose scores a workgroup holds in the L
 constexpr int kScoreKeys = 8;    // keys a wave has in flight
 
 template <int RPL>
-__global__ __launch_bounds__(256) void window_scores_kernel(const float* q, int ldq, int H, int G, int D, int V, float scale, int window,
-                                                            int keep, const int* row_pos, const int* row_slot, const int* page_table, int max_pages,
+__global__ __launch_bounds__(256) void window_scores_kernel(const float* q, int ldq, int H, int G, int D, int V, float scale, KeyMask mask, const int* row_pos, const int* row_slot, const int* page_table, int max_pages,
                                                             int page_tokens, const float* cache, float* sc, int NK, float* st,
                                                             const ScoreShape shape) {
     extern __shared__ __attribute__((aligned(16))) float s_sc[];
@@ -419,7 +425,7 @@ __global__ __launch_bounds__(256) void window_scores_kernel(const float* q, int 
     const int split = blockIdx.x, n_split = gridDim.x, m = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int pos = row_pos[m];
     int k0, k1;
-    const KeySpan span = window_range(pos, window, keep, n_split, split, k0, k1);
+    const KeySpan span = window_range(pos, mask, n_split, split, k0, k1);
     const int* pages = page_table + (size_t)row_slot[m] * max_pages;
     const int rep = H / G;
     const size_t cstride = (size_t)G * (D + V);
@@ -514,8 +520,7 @@ __device__ __forceinline__ bool rows_find_block(int id, const int* ent_len, int 
 }
 
 template <int DH>
-__global__ __launch_bounds__(256) void window_scores_mfma_kernel(const float* q, int ldq, int H, int G, int D, int V, float scale, int window,
-                                                                 int keep, const int* ent_start, const int* ent_len, int n_entries, const int* row_pos,
+__global__ __launch_bounds__(256) void window_scores_mfma_kernel(const float* q, int ldq, int H, int G, int D, int V, float scale, KeyMask mask, const int* ent_start, const int* ent_len, int n_entries, const int* row_pos,
                                                                  const int* row_slot, const int* page_table, int max_pages, int page_tokens,
                                                                  const float* cache, float* sc, int NK, const ScoreShape shape) {
     int e, b;
@@ -525,7 +530,7 @@ __global__ __launch_bounds__(256) void window_scores_mfma_kernel(const float* q,
     const int pos0 = row_pos[m0], pos_last = pos0 + nrows - 1;
     // the block's keys, numbered like a row's: the kept tokens in front of the FIRST row's window, then everything from there to
     // the last row's position (a superset of every row's keys; each pair is masked by its own row's span below)
-    const KeySpan blk = key_span(pos0, window, keep);
+    const KeySpan blk = key_span(pos0, mask);
     const int n_blk = blk.n_first + pos_last - blk.j_lo + 1;
     const int n_tiles = (n_blk - 1) / 32 + 1, units = n_tiles * G;
     const int* pages = page_table + (size_t)row_slot[m0] * max_pages;
@@ -575,7 +580,7 @@ __global__ __launch_bounds__(256) void window_scores_mfma_kernel(const float* q,
             for (int i = 0; i < 16; ++i) {
                 const int qi = 8 * (i >> 2) + 4 * kh + (i & 3);
                 const int pi = pos0 + qi;
-                const KeySpan sp = key_span(pi, window, keep);
+                const KeySpan sp = key_span(pi, mask);
                 if (qi < nrows && j <= pi && (j >= sp.j_lo || j < sp.n_first))
                     sc[((size_t)(m0 + qi) * H + h) * NK + (j >= sp.j_lo ? sp.n_first + (j - sp.j_lo) : j)] = shape_score(acc[i] * scale, shape, h, pi - j);
             }
@@ -585,11 +590,11 @@ __global__ __launch_bounds__(256) void window_scores_mfma_kernel(const float* q,
 
 // Per row and head the maximum and the sum of exp of the row's scores (a wave per head, its lanes over the keys), filed as the
 // statistics of share 0; the other shares are marked empty.
-__global__ __launch_bounds__(256) void window_stats_kernel(const float* sc, int NK, int H, int window, int keep, int n_split, const int* row_pos,
+__global__ __launch_bounds__(256) void window_stats_kernel(const float* sc, int NK, int H, KeyMask mask, int n_split, const int* row_pos,
                                                            float* st) {
     const int m = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int pos = row_pos[m];
-    const int n_keys = key_span(pos, window, keep).n_keys;
+    const int n_keys = key_span(pos, mask).n_keys;
     for (int h = wave; h < H; h += 4) {
         const float* sr = sc + ((size_t)m * H + h) * NK;
         float mx = -INFINITY;
@@ -606,7 +611,7 @@ __global__ __launch_bounds__(256) void window_stats_kernel(const float* sc, int 
     }
 }
 
-__global__ __launch_bounds__(256) void window_mix_kernel(int H, int G, int D, int V, int window, int keep, const float* sink, const float* talk,
+__global__ __launch_bounds__(256) void window_mix_kernel(int H, int G, int D, int V, KeyMask mask, const float* sink, const float* talk,
                                                          const int* row_pos, const int* row_slot, const int* page_table, int max_pages,
                                                          int page_tokens, const float* cache, const float* sc, int NK, const float* st,
                                                          float* po) {
@@ -620,7 +625,7 @@ __global__ __launch_bounds__(256) void window_mix_kernel(int H, int G, int D, in
     const int split = blockIdx.x, n_split = gridDim.x, m = blockIdx.y, tid = threadIdx.x;
     const int pos = row_pos[m];
     int k0, k1;
-    const KeySpan span = window_range(pos, window, keep, n_split, split, k0, k1);
+    const KeySpan span = window_range(pos, mask, n_split, split, k0, k1);
     const int* pages = page_table + (size_t)row_slot[m] * max_pages;
     const int rep = H / G;
     const size_t cstride = (size_t)G * (D + V);
@@ -702,7 +707,7 @@ constexpr int kPvHeads = 16; // most heads a workgroup weighs (a pair's weights 
 // pv_block_heads of them), so any number of heads fits and no score is read by more than one group of units.
 __host__ __device__ constexpr int pv_block_heads(int ctiles) { return (4 * kPvUnits - 1) / ctiles + 2; }
 
-__global__ __launch_bounds__(256) void window_mix_mfma_kernel(int H, int G, int D, int V, int window, int keep, const float* sink, const float* talk,
+__global__ __launch_bounds__(256) void window_mix_mfma_kernel(int H, int G, int D, int V, KeyMask mask, const float* sink, const float* talk,
                                                               const int* ent_start, const int* ent_len, int n_entries, const int* row_pos,
                                                               const int* row_slot, const int* page_table, int max_pages, int page_tokens,
                                                               const float* cache, const float* sc, int NK, const float* st, int n_split,
@@ -725,7 +730,7 @@ __global__ __launch_bounds__(256) void window_mix_mfma_kernel(int H, int G, int 
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 31, kh = lane >> 5;
     const int m0 = ent_start[e] + 32 * b, nrows = min(32, ent_len[e] - 32 * b);
     const int pos0 = row_pos[m0], pos_last = pos0 + nrows - 1;
-    const KeySpan blk = key_span(pos0, window, keep);  // the block's keys, numbered as in window_scores_mfma_kernel
+    const KeySpan blk = key_span(pos0, mask);  // the block's keys, numbered as in window_scores_mfma_kernel
     const int n_blk = blk.n_first + pos_last - blk.j_lo + 1;
     const int n_tiles = (n_blk - 1) / kPvKeys + 1, per = (n_tiles + gridDim.y - 1) / gridDim.y;
     const int t_lo = min(n_tiles, (int)blockIdx.y * per), t_hi = min(n_tiles, t_lo + per);
@@ -762,7 +767,7 @@ __global__ __launch_bounds__(256) void window_mix_mfma_kernel(int H, int G, int 
         for (int pr = tid; pr < 32 * kPvKeys; pr += blockDim.x) {
             const int row = pr / kPvKeys, kk = pr % kPvKeys, pi = pos0 + row;
             const int j = n0 + kk < n_blk ? key_pos(blk, n0 + kk) : pos_last + 1;
-            const KeySpan sp = key_span(pi, window, keep);
+            const KeySpan sp = key_span(pi, mask);
             const bool ok = row < nrows && j <= pi && (j >= sp.j_lo || j < sp.n_first);
             float p[kPvHeads];  // (registers: the loops over it are unrolled to the kernel's most heads)
             const float* sr = sc + ((size_t)(m0 + min(row, nrows - 1)) * H + h_lo) * NK + (ok ? (j >= sp.j_lo ? sp.n_first + (j - sp.j_lo) : j) : 0);
@@ -1272,7 +1277,7 @@ int launch_norm_conv_single(float* x, const float* x0, const float* yl, const fl
 int launch_window_prep(float* proj, int ld, int M, int H, int G, int D, int V, Rotary rot, const float* vfreq, const int* row_pos,
                        const int* row_slot, const int* page_table, int max_pages, int page_tokens, float* cache, hipStream_t s) {
     if (M <= 0) return ZG_OK;
-    ZG_REQUIRE(V % 2 == 0 && rot.dims % 2 == 0 && rot.dims <= D, ZG_ERR_ARG, "windowed attention: %d value channels, %d of %d rotated", V, rot.dims, D);
+    ZG_REQUIRE((!vfreq || V % 2 == 0) && rot.dims % 2 == 0 && rot.dims <= D, ZG_ERR_ARG, "windowed attention: %d value channels, %d of %d rotated", V, rot.dims, D);
     window_prep_kernel<<<M, 256, 0, s>>>(proj, ld, H, G, D, V, rot, vfreq, row_pos, row_slot, page_table, max_pages, page_tokens, cache);
     ZG_HIP(hipGetLastError());
     return ZG_OK;
@@ -1298,8 +1303,7 @@ int launch_whole_norm_prep(float* qkv, int ld, int M, int HD, int GD, int GV, co
     return ZG_OK;
 }
 
-int launch_window_attention(const float* q, int ldq, float* out, int ldo, int M, int H, int G, int D, int V, float scale, int window,
-                            int keep_first, const float* sink, const float* talk, const float* vfreq, const int* row_pos, const int* row_slot,
+int launch_window_attention(const float* q, int ldq, float* out, int ldo, int M, int H, int G, int D, int V, float scale, KeyMask mask, const float* sink, const float* talk, const float* vfreq, const int* row_pos, const int* row_slot,
                             const int* page_table, int max_pages, int page_tokens, const float* cache, hipStream_t s, ScoreShape shape) {
     if (M <= 0) return ZG_OK;
     ZG_REQUIRE(H >= 1 && H <= kWinMaxHeads && G >= 1 && H % G == 0, ZG_ERR_UNSUPPORTED, "windowed attention: %d heads on %d key heads (at most %d heads)",
@@ -1308,7 +1312,8 @@ int launch_window_attention(const float* q, int ldq, float* out, int ldo, int M,
                256 * kWinAcc);
     const size_t lds = ((size_t)H * D + 2 * (size_t)H * kWinTile + (size_t)H * H + (size_t)H * V) * sizeof(float);
     ZG_REQUIRE(lds <= 60 * 1024, ZG_ERR_UNSUPPORTED, "windowed attention: %d heads of %d + %d channels need %zu bytes of LDS", H, D, V, lds);
-    window_attention_kernel<<<M, 256, lds, s>>>(q, ldq, out, ldo, H, G, D, V, scale, window, window > 0 ? keep_first : 0, sink, talk, vfreq, row_pos, row_slot, page_table,
+    if (mask.window <= 0) mask.keep = 0;
+    window_attention_kernel<<<M, 256, lds, s>>>(q, ldq, out, ldo, H, G, D, V, scale, mask, sink, talk, vfreq, row_pos, row_slot, page_table,
                                                 max_pages, page_tokens, cache, shape);
     ZG_HIP(hipGetLastError());
     return ZG_OK;
@@ -1331,14 +1336,13 @@ size_t window_split_workspace(int rows, int H, int V, int key_capacity, int* n_s
     return (size_t)rows * H * key_capacity + (size_t)rows * n_split * H * 2 + (size_t)rows * n_split * H * V;
 }
 
-int launch_window_attention_split(const float* q, int ldq, float* out, int ldo, int M, int H, int G, int D, int V, float scale, int window,
-                                  int keep_first, const float* sink, const float* talk, const float* vfreq, const int* row_pos, const int* row_slot,
+int launch_window_attention_split(const float* q, int ldq, float* out, int ldo, int M, int H, int G, int D, int V, float scale, KeyMask mask, const float* sink, const float* talk, const float* vfreq, const int* row_pos, const int* row_slot,
                                   const int* page_table, int max_pages, int page_tokens, const float* cache, int key_capacity, float* ws,
                                   size_t ws_floats, const int* ent_start, const int* ent_len, int n_entries, hipStream_t s, bool* taken,
                                   const float* out_gate, int ld_gate, float out_factor, ScoreShape shape) {
     *taken = false;
     if (M <= 0) return ZG_OK;
-    const int keep = window > 0 ? keep_first : 0;
+    if (mask.window <= 0) mask.keep = 0;
     if (const char* e = getenv("ZGPT2_LM_WINDOW_GENERAL"))  // test hook: every step through the general kernel
         if (atoi(e) != 0) return ZG_OK;
     int n_split = 1;
@@ -1363,7 +1367,7 @@ int launch_window_attention_split(const float* q, int ldq, float* out, int ldo, 
         const int ksplit = std::max(1, std::min(16, (max_tiles * G + 7) / 8));
         const dim3 tg((M + 31) / 32 + n_entries, ksplit);
 #define ZG_WT(R)                                                                                                                                   \
-    window_scores_mfma_kernel<R><<<tg, 256, 0, s>>>(q, ldq, H, G, D, V, scale, window, keep, ent_start, ent_len, n_entries, row_pos, row_slot, page_table, \
+    window_scores_mfma_kernel<R><<<tg, 256, 0, s>>>(q, ldq, H, G, D, V, scale, mask, ent_start, ent_len, n_entries, row_pos, row_slot, page_table, \
                                                     max_pages, page_tokens, cache, sc, key_capacity, shape)
         if (dh <= 8) ZG_WT(8);
         else if (dh <= 16) ZG_WT(16);
@@ -1371,11 +1375,11 @@ int launch_window_attention_split(const float* q, int ldq, float* out, int ldo, 
         else ZG_WT(64);
 #undef ZG_WT
         ZG_HIP(hipGetLastError());
-        window_stats_kernel<<<M, 256, 0, s>>>(sc, key_capacity, H, window, keep, n_split, row_pos, st);
+        window_stats_kernel<<<M, 256, 0, s>>>(sc, key_capacity, H, mask, n_split, row_pos, st);
         ZG_HIP(hipGetLastError());
     } else {
 #define ZG_WS(R)                                                                                                                              \
-    window_scores_kernel<R><<<grid, 256, lds_a, s>>>(q, ldq, H, G, D, V, scale, window, keep, row_pos, row_slot, page_table, max_pages, page_tokens, cache, \
+    window_scores_kernel<R><<<grid, 256, lds_a, s>>>(q, ldq, H, G, D, V, scale, mask, row_pos, row_slot, page_table, max_pages, page_tokens, cache, \
                                                      sc, key_capacity, st, shape)
     if (rpl <= 1) ZG_WS(1);
     else if (rpl <= 2) ZG_WS(2);
@@ -1389,10 +1393,10 @@ int launch_window_attention_split(const float* q, int ldq, float* out, int ldo, 
     if (tiled && (!mixes || H <= kPvHeads) && lds_c <= 60 * 1024) {  // the value product of 32 rows at a time on the matrix cores
         const int units = H * ((V + 31) / 32);
         const dim3 pg((M + 31) / 32 + n_entries, n_split, (units + 4 * kPvUnits - 1) / (4 * kPvUnits));
-        window_mix_mfma_kernel<<<pg, 256, lds_c, s>>>(H, G, D, V, window, keep, sink, talk, ent_start, ent_len, n_entries, row_pos, row_slot, page_table,
+        window_mix_mfma_kernel<<<pg, 256, lds_c, s>>>(H, G, D, V, mask, sink, talk, ent_start, ent_len, n_entries, row_pos, row_slot, page_table,
                                                       max_pages, page_tokens, cache, sc, key_capacity, st, n_split, po);
     } else {
-        window_mix_kernel<<<grid, 256, lds_b, s>>>(H, G, D, V, window, keep, sink, talk, row_pos, row_slot, page_table, max_pages, page_tokens, cache, sc,
+        window_mix_kernel<<<grid, 256, lds_b, s>>>(H, G, D, V, mask, sink, talk, row_pos, row_slot, page_table, max_pages, page_tokens, cache, sc,
                                                    key_capacity, st, po);
     }
     ZG_HIP(hipGetLastError());

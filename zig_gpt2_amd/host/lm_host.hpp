@@ -160,10 +160,11 @@ typedef std::vector<std::pair<std::string, std::vector<float>>> DerivedTensors;
 inline void build_config(const Json& cfg, const Json* tensors, std::vector<zg_lm_layer>& layers, zg_lm_config& out, DerivedTensors* derived = nullptr) {
     const Json* arch = cfg.get("architecture");
     const std::string design = arch ? arch->str : std::string("?");
-    if (design != "Tokosun" && design != "Gupizen" && design != "Sanazen" && design != "Vovalorn")
+    if (design != "Tokosun" && design != "Gupizen" && design != "Sanazen" && design != "Vovalorn" && design != "Duvulix")
         throw std::runtime_error("config: architecture '" + design + "' is not served");
-    const bool gup = design == "Gupizen", san = design == "Sanazen", vov = design == "Vovalorn";
+    const bool gup = design == "Gupizen", san = design == "Sanazen", vov = design == "Vovalorn", duv = design == "Duvulix";
     memset(&out, 0, sizeof(out));
+    if (duv) out.flags |= ZG_LM_NO_SHIFT;  // what the name fixes: the mixer reads the norm as it is
     if (vov) {  // what the name fixes: norms without statistics, one of them behind the embedding
         out.flags |= ZG_LM_TANH_NORMS | ZG_LM_EMBED_NORM;
         out.residual_mult = 1.0f;
@@ -222,8 +223,23 @@ inline void build_config(const Json& cfg, const Json* tensors, std::vector<zg_lm
         const std::string prefix = "l" + std::to_string(own) + ".";
         const Json& sizes = ((gup || san) && type == "parallel") ? m.at("left") : m;
         d.heads = (int)sizes.at("heads").num;
-        d.dim = (int)sizes.at("dim").num;
+        d.dim = (int)sizes.at(duv && type == "mamba2" ? "state" : "dim").num;
         d.vdim = sizes.get("vdim") ? (int)sizes.at("vdim").num : d.dim;
+        if (duv) d.rot_halves = 1;
+        auto yarn_rotary = [&] {
+            d.rot_base = 10000.0f;
+            const Json* rot = m.get("rot");
+            if (!rot || !rot->truthy()) return;
+            if (const Json* v = rot->get("dims")) d.rot_dims = (int)v->num;
+            if (const Json* v = rot->get("base")) d.rot_base = (float)v->num;
+            const Json* sc = rot->get("scaling");
+            if (!sc || !sc->truthy()) return;
+            d.rot_scaled = ZG_LM_ROT_YARN;
+            d.rot_factor = (float)sc->at("factor").num;
+            d.rot_original = (float)sc->at("original").num;
+            d.rot_fast = (float)sc->at("fast").num;
+            d.rot_slow = (float)sc->at("slow").num;
+        };
         if (gup) {
             d.ff_act = ZG_LM_ACT_GELU;
             d.router = ZG_LM_ROUTE_TOP_LOGITS;
@@ -323,29 +339,37 @@ inline void build_config(const Json& cfg, const Json* tensors, std::vector<zg_lm
             if (const Json* v = m.get("dist_bias")) d.dist_bias = v->truthy() ? 1 : 0;
         } else if (vov) {
             throw std::runtime_error("config: unknown mixer type '" + type + "'");
+        } else if (duv && type == "attention") {
+            d.mixer = ZG_LM_MIX_ROTARY_ATTENTION;
+            d.kv_heads = m.get("kv_heads") ? (int)m.at("kv_heads").num : d.heads;
+            d.scale = (float)m.at("scale").num;
+            if (const Json* mask = m.get("mask"))
+                if (mask->truthy())
+                    if (const Json* v = mask->get("size")) d.chunk = (int)v->num;
+            yarn_rotary();
+        } else if (duv && type == "mamba2") {
+            d.mixer = ZG_LM_MIX_SSD;
+            d.kv_heads = m.get("groups") ? (int)m.at("groups").num : 1;
+            d.conv = (int)m.at("conv").num;
+            d.norm_groups = m.get("norm_groups") ? (int)m.at("norm_groups").num : 1;
+        } else if (duv && type != "latent_attention") {
+            throw std::runtime_error("config: unknown mixer type '" + type + "'");
         } else if (type == "hgrn2") {
             d.mixer = ZG_LM_MIX_HGRN2;
         } else if (type == "latent_attention") {
             d.mixer = ZG_LM_MIX_LATENT_ATTENTION;
             d.rot_dim = (int)m.at("rot_dim").num;
             d.kv_rank = (int)m.at("kv_rank").num;
-            d.q_rank = (int)m.at("q_rank").num;
+            if (duv) {  // queries projected directly, a gate per head, latents possibly another layer's
+                d.head_gate = 1;
+                if (const Json* v = m.get("kv_from"))
+                    if (v->kind == Json::Num) d.kv_from = (int)v->num + 1;
+            } else {
+                d.q_rank = (int)m.at("q_rank").num;
+            }
             d.scale = (float)m.at("scale").num;
             d.rot_dims = d.rot_dim;
-            d.rot_base = 10000.0f;
-            if (const Json* rot = m.get("rot"))
-                if (rot->truthy()) {
-                    if (const Json* v = rot->get("dims")) d.rot_dims = (int)v->num;
-                    if (const Json* v = rot->get("base")) d.rot_base = (float)v->num;
-                    const Json* sc = rot->get("scaling");
-                    if (sc && sc->truthy()) {
-                        d.rot_scaled = 1;
-                        d.rot_factor = (float)sc->at("factor").num;
-                        d.rot_original = (float)sc->at("original").num;
-                        d.rot_fast = (float)sc->at("fast").num;
-                        d.rot_slow = (float)sc->at("slow").num;
-                    }
-                }
+            yarn_rotary();
         } else {
             throw std::runtime_error("config: unknown mixer type '" + type + "'");
         }
@@ -355,6 +379,7 @@ inline void build_config(const Json& cfg, const Json* tensors, std::vector<zg_lm
             if (kind == "dense") {
                 d.ff = ZG_LM_FF_DENSE;
                 d.ff_width = (int)mlp->at("ff").num;
+                if (duv) d.dense_act = ZG_LM_DENSE_POLYNORM;
             } else if (kind == "moe") {
                 d.ff = ZG_LM_FF_MOE;
                 d.ff_width = (int)mlp->at("expert").at("ff").num;

@@ -30,6 +30,10 @@ config.json (zig_gpt2_amd/models.py maps architecture names to loaders; `DESIGNS
   `<name>.alpha`), also behind the embedding (`embed.norm`); residual_mult: factor of every sublayer's normed output in the
   residual sum; experts chosen by sigmoid scores + correction among the best contiguous blocks of experts (router.groups:
   count, keep), weights normalised over the chosen, times router.scale; mlp.shared: an expert every token uses.
+  Duvulix: type "latent_attention" (queries projected directly, rotary pairs (i, i + dims / 2), every head gated by sigmoid(W_g h)_h;
+  kv_from: j: the layer reads layer j's latents instead of making its own) | "attention" (grouped-query attention, rotary with
+  YaRN scaling; a query sees its own chunk of mask.size positions) | "mamba2" (selective state space: heads, vdim, state, groups,
+  conv, norm_groups); the mixer reads norm1(x) as it is; dense feed-forwards with a polynomial activation (tensor mlp.act).
 """
 import ctypes as C
 import json
@@ -44,7 +48,8 @@ from ._lib import check_lm as check
 
 MIXERS = {"hgrn2": _lib.LM_MIX_HGRN2, "latent_attention": _lib.LM_MIX_LATENT_ATTENTION, "parallel": _lib.LM_MIX_PARALLEL,
           "channel_delta": _lib.LM_MIX_CHANNEL_DELTA, "window_linear": _lib.LM_MIX_WINDOW_LINEAR, "gla": _lib.LM_MIX_GLA,
-          "attention": _lib.LM_MIX_ATTENTION}
+          "attention": _lib.LM_MIX_ATTENTION, "rotary_attention": _lib.LM_MIX_ROTARY_ATTENTION, "ssd": _lib.LM_MIX_SSD}
+DENSE_ACTS = {"relu2": _lib.LM_DENSE_RELU2, "polynorm": _lib.LM_DENSE_POLYNORM}
 ROT_STYLES = {"yarn": _lib.LM_ROT_YARN, "bands": _lib.LM_ROT_BANDS}
 EXPERT_ACTS = {"glu_silu": _lib.LM_ACT_GLU_SILU, "gelu": _lib.LM_ACT_GELU, "glu_clipped": _lib.LM_ACT_GLU_CLIPPED}
 ROUTERS = {"softmax_all": _lib.LM_ROUTE_SOFTMAX_ALL, "top_logits": _lib.LM_ROUTE_TOP_LOGITS, "sigmoid_input": _lib.LM_ROUTE_SIGMOID_INPUT,
@@ -61,6 +66,8 @@ DESIGNS = {
                     side_by_side=True, sinusoid_positions=True),
     "Vovalorn": dict(mixers={"gla": "gla", "attention": "attention"}, tied_head=False, loop_readd=False, expert_act="glu_silu", router="sigmoid_groups",
                      tanh_norms=True, embed_norm=True),
+    "Duvulix": dict(mixers={"latent_attention": "latent_attention", "attention": "rotary_attention", "mamba2": "ssd"}, tied_head=False, loop_readd=False,
+                    expert_act="glu_silu", router="softmax_all", no_shift=True, dense_act="polynorm", rot_halves=True, direct_queries=True),
 }
 
 
@@ -113,6 +120,12 @@ class LayerSpec:
     route_keep: int = 1
     route_scale: float = 1.0
     weights_of: Optional[int] = None  # this layer runs the tensors of that layer
+    rot_halves: bool = False  # rotary pairs (i, i + dims / 2) instead of (2i, 2i + 1)
+    chunk: int = 0  # rotary attention: a query sees its own chunk of this many positions (0: no chunks)
+    kv_from: Optional[int] = None  # latent attention: the latents of that layer
+    head_gate: bool = False  # latent attention: head h times sigmoid(W_g h)_h
+    norm_groups: int = 0  # ssd: parts of the norm behind the gate (ssd: dim = state rows, kv_heads = groups of B and C)
+    dense_act: str = "relu2"
 
     @classmethod
     def from_json(cls, entry, design="Tokosun", shapes=None, prefix=""):
@@ -164,18 +177,30 @@ class LayerSpec:
         elif kind == "channel_delta":
             kw = dict(mixer=kind, heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=int(m["dim"]), vdim=int(m["vdim"]),
                       conv=int(m["conv"]), decay_rank=inner("decay_rank", "mix.a1"), gate_rank=inner("gate_rank", "mix.g1"))
+        elif kind == "rotary_attention":
+            rot = m.get("rot") or {}
+            kw = dict(mixer=kind, heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=int(m["dim"]),
+                      vdim=int(m.get("vdim", m["dim"])), scale=float(m["scale"]), chunk=int((m.get("mask") or {}).get("size", 0)),
+                      rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 10000.0)),
+                      rot_scaling=dict(rot["scaling"]) if rot.get("scaling") else None)
+        elif kind == "ssd":
+            kw = dict(mixer=kind, heads=int(m["heads"]), vdim=int(m["vdim"]), dim=int(m["state"]), kv_heads=int(m.get("groups", 1)), conv=int(m["conv"]),
+                      norm_groups=int(m.get("norm_groups", 1)))
         else:
             kw = dict(mixer=kind, heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]))
+        kw.update(rot_halves=bool(fixed.get("rot_halves")))
         kw.update(expert_act=fixed["expert_act"], router=fixed["router"])
         if kind == "latent_attention":
             rot = m.get("rot") or {}
-            kw.update(rot_dim=int(m["rot_dim"]), kv_rank=int(m["kv_rank"]), q_rank=int(m["q_rank"]), scale=float(m["scale"]),
+            direct = bool(fixed.get("direct_queries"))
+            kw.update(head_gate=direct, kv_from=int(m["kv_from"]) if m.get("kv_from") is not None else None)
+            kw.update(rot_dim=int(m["rot_dim"]), kv_rank=int(m["kv_rank"]), q_rank=0 if direct else int(m["q_rank"]), scale=float(m["scale"]),
                       rot_dims=int(rot.get("dims", m["rot_dim"])), rot_base=float(rot.get("base", 10000.0)),
                       rot_scaling=dict(rot["scaling"]) if rot.get("scaling") else None)
         mlp = entry.get("mlp")
         if mlp:
             if mlp["kind"] == "dense":
-                kw.update(ff="dense", ff_width=int(mlp["ff"]))
+                kw.update(ff="dense", ff_width=int(mlp["ff"]), dense_act=fixed.get("dense_act", "relu2"))
             elif mlp["kind"] == "moe":
                 kw.update(ff="moe", ff_width=int(mlp["expert"]["ff"]), experts=int(mlp["router"]["experts"]), top=int(mlp["router"]["top"]))
                 if fixed["expert_act"] == "glu_clipped":
@@ -216,7 +241,21 @@ class LayerSpec:
             rot = {"base": self.rot_base, "dims": self.rot_dims}
             if self.rot_scaling:
                 rot["scaling"] = dict(self.rot_scaling)
-            mixer.update(rot_dim=self.rot_dim, kv_rank=self.kv_rank, q_rank=self.q_rank, scale=self.scale, rot=rot)
+            mixer.update(rot_dim=self.rot_dim, kv_rank=self.kv_rank, scale=self.scale, rot=rot)
+            if self.q_rank:
+                mixer["q_rank"] = self.q_rank
+            if self.kv_from is not None:
+                mixer["kv_from"] = self.kv_from
+        if self.mixer == "rotary_attention":
+            mixer.update(kv_heads=self.kv_heads, scale=self.scale)
+            if self.rot_dims:
+                mixer["rot"] = {"base": self.rot_base, "dims": self.rot_dims}
+                if self.rot_scaling:
+                    mixer["rot"]["scaling"] = dict(self.rot_scaling)
+            if self.chunk:
+                mixer["mask"] = {"size": self.chunk}
+        elif self.mixer == "ssd":
+            mixer = {"heads": self.heads, "vdim": self.vdim, "state": self.dim, "groups": self.kv_heads, "conv": self.conv, "norm_groups": self.norm_groups}
         if self.mixer == "gla":
             mixer.update(tau=self.tau, decay_rank=self.decay_rank)
         elif self.mixer == "attention":
@@ -239,7 +278,8 @@ class LayerSpec:
                 mlp["shared"] = {"ff": self.shared_width}
             if self.router == "sigmoid_groups":
                 mlp["router"].update(groups={"count": self.route_groups, "keep": self.route_keep}, scale=self.route_scale)
-        out = {"type": "parallel" if self.mixer == "window_linear" else self.mixer, "mixer": mixer, "mlp": mlp}
+        kinds = {"window_linear": "parallel", "rotary_attention": "attention", "ssd": "mamba2"}  # config.json's names where they differ
+        out = {"type": kinds.get(self.mixer, self.mixer), "mixer": mixer, "mlp": mlp}
         if self.weights_of is not None:
             out["weights_of"] = self.weights_of
         return out
@@ -256,9 +296,10 @@ class LayerSpec:
                             self.gate_rank, EXPERT_ACTS[self.expert_act], ROUTERS[self.router], self.keep_first, self.left_scale, self.right_scale,
                             self.lin_heads, self.lin_dim, self.lin_vdim, self.ff_limit, self.shared_width, self.shared_limit, self.tau, self.softcap,
                             self.qtemp_coef, self.qtemp_every, int(self.dist_bias), self.route_groups, self.route_keep, self.route_scale,
-                            0 if self.weights_of is None else self.weights_of + 1)
+                            0 if self.weights_of is None else self.weights_of + 1, int(self.rot_halves), self.chunk,
+                            0 if self.kv_from is None else self.kv_from + 1, int(self.head_gate), self.norm_groups, DENSE_ACTS[self.dense_act])
 
-    def tensor_shapes(self, prefix, width, canon_taps=0, tanh_norms=False):
+    def tensor_shapes(self, prefix, width, canon_taps=0, tanh_norms=False, no_shift=False):
         """{checkpoint tensor name: shape} of this layer (none for a layer that runs another layer's tensors)."""
         if self.weights_of is not None:
             return {}
@@ -266,7 +307,7 @@ class LayerSpec:
         t = {prefix + "norm1": (W,), prefix + "norm1b": (W,)}
         if self.mixer == "window_linear":  # plain norms in front of the sublayers only, nothing between norm and mixer
             t = {prefix + "norm1": (W,)}
-        elif tanh_norms:  # the mixer reads the norm as it is
+        elif tanh_norms or no_shift:  # the mixer reads the norm as it is
             pass
         elif canon_taps:
             t[prefix + "canon1"] = (W, canon_taps)
@@ -309,8 +350,21 @@ class LayerSpec:
                       m + "o": (W, H * V)})
         elif self.mixer == "latent_attention":
             R, KR, QR = self.rot_dim, self.kv_rank, self.q_rank
-            t.update({m + "dq": (QR, W), m + "dq.norm": (QR,), m + "uq": (H * (D + R), QR), m + "dkv": (KR + R, W), m + "dkv.norm": (KR,),
-                      m + "uk": (H * D, KR), m + "uv": (H * V, KR), m + "o": (W, H * V)})
+            t.update({m + "uk": (H * D, KR), m + "uv": (H * V, KR), m + "o": (W, H * V)})
+            if QR:
+                t.update({m + "dq": (QR, W), m + "dq.norm": (QR,), m + "uq": (H * (D + R), QR)})
+            else:
+                t[m + "q"] = (H * (D + R), W)
+            if self.kv_from is None:
+                t.update({m + "dkv": (KR + R, W), m + "dkv.norm": (KR,)})
+            if self.head_gate:
+                t[m + "g"] = (H, W)
+        elif self.mixer == "rotary_attention":
+            t.update({m + "q": (H * D, W), m + "k": (self.kv_heads * D, W), m + "v": (self.kv_heads * V, W), m + "o": (W, H * V)})
+        elif self.mixer == "ssd":
+            inner, bc = H * V, 2 * self.kv_heads * D
+            t.update({m + "in": (2 * inner + bc + H, W), m + "conv": (inner + bc, self.conv), m + "conv.b": (inner + bc,), m + "dt_bias": (H,),
+                      m + "A_log": (H,), m + "D": (H,), m + "norm": (inner,), m + "o": (W, inner)})
         f = prefix + "mlp."
         if self.ff != "none":
             t.update({prefix + "norm2": (W,), prefix + "norm2b": (W,)})
@@ -318,6 +372,8 @@ class LayerSpec:
                 del t[prefix + "norm2b"]
         if self.ff == "dense":
             t.update({f + "up": (self.ff_width, W), f + "down": (W, self.ff_width)})
+            if self.dense_act == "polynorm":
+                t[f + "act"] = (4,)
         elif self.ff == "moe":
             for e in range(self.experts):
                 t.update({f"{f}e{e}.up": (self.ff_width, W), f"{f}e{e}.down": (W, self.ff_width)})
@@ -405,7 +461,7 @@ class LMConfig:
             out["logit_softcap"] = self.logit_softcap
         if self.residual_mult != 1.0:
             out["residual_mult"] = self.residual_mult
-        if out["loop"] is None and DESIGNS[self.architecture].get("tanh_norms"):
+        if out["loop"] is None and (DESIGNS[self.architecture].get("tanh_norms") or DESIGNS[self.architecture].get("no_shift")):
             del out["loop"]
         return out
 
@@ -417,7 +473,8 @@ class LMConfig:
         d = DESIGNS[self.architecture]
         return ((_lib.LM_TIED_HEAD if d["tied_head"] else 0) | (_lib.LM_LOOP_READD if d["loop_readd"] else 0) |
                 (_lib.LM_SIDE_BY_SIDE if d.get("side_by_side") else 0) | (_lib.LM_SINUSOID_POSITIONS if d.get("sinusoid_positions") else 0) |
-                (_lib.LM_TANH_NORMS if d.get("tanh_norms") else 0) | (_lib.LM_EMBED_NORM if d.get("embed_norm") else 0))
+                (_lib.LM_TANH_NORMS if d.get("tanh_norms") else 0) | (_lib.LM_EMBED_NORM if d.get("embed_norm") else 0) |
+                (_lib.LM_NO_SHIFT if d.get("no_shift") else 0))
 
     def passes(self):
         """Layer index of every pass, in execution order."""
@@ -438,7 +495,7 @@ class LMConfig:
         if not self.tied_head:
             t["head"] = (self.vocab, self.width)
         for i, l in enumerate(self.layers):
-            t.update(l.tensor_shapes(f"l{i}.", self.width, self.canon_taps, tanh_norms))
+            t.update(l.tensor_shapes(f"l{i}.", self.width, self.canon_taps, tanh_norms, bool(d.get("no_shift"))))
         return t
 
     def derived_tensors(self):
