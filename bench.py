@@ -48,10 +48,11 @@ def parse():
                    help="instead of the default workload: prompt and decode throughput of a layered model (Tokosun design, random weights) "
                         "at a size that resembles GPT-2 124M / medium / XL, beside the GPT-2 model of the same width and depth")
     p.add_argument("--lm-dtype", default="bfloat16", choices=["bfloat16", "float32"])
-    p.add_argument("--lm-design", default="tokosun", choices=["tokosun", "gupizen", "sanazen", "vovalorn"],
+    p.add_argument("--lm-design", default="tokosun", choices=["tokosun", "gupizen", "sanazen", "vovalorn", "duvulix"],
                    help="with --lm: which design is measured.  gupizen: a Gupizen stack of the same width and depth, beside the Tokosun stack "
                         "(the tier's closest model) instead of GPT-2.  sanazen: a Sanazen stack beside the Gupizen stack of the same width and depth.  "
-                        "vovalorn: a Vovalorn stack beside the Tokosun stack of the same width and depth")
+                        "vovalorn: a Vovalorn stack beside the Tokosun stack of the same width and depth; "
+                        "duvulix: a Duvulix stack beside the Tokosun stack of the same width and depth")
     p.add_argument("--dry-run", action="store_true",
                    help="CPU rehearsal of the launch path (gloo, no GPU, no kernels): rendezvous, prompt sharding, "
                         "weight-arena broadcast, barriers and the max-reduce; prints a line with dry_run=true")
@@ -504,6 +505,25 @@ def vovalorn_bench_config(width, n_layers, vocab):
                        architecture="Vovalorn", residual_mult=0.5)
 
 
+def duvulix_bench_config(width, n_layers, vocab, chunk=512):
+    """A Duvulix-design stack of `n_layers` layers in the repeating order state space, latent attention, latent attention that reads the
+    latents of the layer before, chunked attention: a state space of 2 x width channels in heads of 64 with a state of 128 rows in
+    one group, latent heads of 64 + 32 channels on latents of 256, attention heads of 64 channels on a quarter (a fifth) as many
+    key heads in chunks of `chunk` positions, every layer with a dense feed-forward of 4 x width."""
+    from zig_gpt2_amd import lm
+
+    heads = width // 64
+    kv = heads // 4 if heads % 4 == 0 else heads // 5 if heads % 5 == 0 else heads
+    dense = dict(ff="dense", ff_width=4 * width, dense_act="polynorm", rot_halves=True)
+    ssm = dict(mixer="ssd", heads=2 * width // 64, vdim=64, dim=128, kv_heads=1, conv=4, norm_groups=1, **dense)
+    lat = dict(mixer="latent_attention", heads=heads, dim=64, vdim=64, rot_dim=32, kv_rank=256, scale=(64 + 32) ** -0.5, rot_dims=32, rot_base=10000.0,
+               head_gate=True, **dense)
+    att = dict(mixer="rotary_attention", heads=heads, kv_heads=kv, dim=64, vdim=64, scale=64 ** -0.5, chunk=chunk, rot_dims=64, rot_base=10000.0,
+               rot_scaling={"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}, **dense)
+    layers = [lm.LayerSpec(**[ssm, lat, dict(lat, kv_from=i - 1), att][i % 4]) for i in range(n_layers)]
+    return lm.LMConfig(vocab=vocab, width=width, layers=layers, norm_eps=1e-6, architecture="Duvulix")
+
+
 def lm_weight_bytes(cfg):
     """(stored, read per decoded token) bytes of the bf16 matrices: every expert is stored, `top` of them are read."""
     stored = active = 0
@@ -531,6 +551,7 @@ def lm_bench(a):
     gup = a.lm_design == "gupizen"
     san = a.lm_design == "sanazen"
     vov = a.lm_design == "vovalorn"
+    duv = a.lm_design == "duvulix"
     cfg = lm_bench_config(width, n_layers, gcfg.vocab_size)
     out = {"metric": "lm_decode_tokens_per_s", "unit": "tokens/s", "n_gpus": 1, "steps": a.steps, "warmup": a.warmup, "higher_is_better": True,
            "scaling": "weak", "vs_baseline": None, "dtype": "bf16" if a.lm_dtype == "bfloat16" else "fp32", "data": "synthetic (random weights, filled on the GPU)",
@@ -599,6 +620,15 @@ def lm_bench(a):
         out["config"]["model"] = (f"Vovalorn design, width {width}, {n_layers} layers (gated linear attention, attention x2, gated linear attention; "
                                   f"8 experts in 2 groups, 2 chosen, one shared), vocab {gcfg.vocab_size}")
         out.update(value=d1["tokens_per_s"], ms_per_step=round(d1["wall_us_per_step"] / 1e3, 4), vovalorn=v_res, tokosun_equal_size=t_res)
+        print(json.dumps(out))
+        return
+    if duv:  # beside the tier's closest model (latent attention and a matrix-state recurrence in sequential sublayers with offset norms)
+        d_res = measure(duvulix_bench_config(width, n_layers, gcfg.vocab_size))
+        t_res = measure(lm_bench_config(width, n_layers, gcfg.vocab_size))
+        d1 = d_res["decode"][0]
+        out["config"]["model"] = (f"Duvulix design, width {width}, {n_layers} layers (state space, latent attention, latent attention on the same "
+                                  f"latents, attention in chunks of 512; dense feed-forwards), vocab {gcfg.vocab_size}")
+        out.update(value=d1["tokens_per_s"], ms_per_step=round(d1["wall_us_per_step"] / 1e3, 4), duvulix=d_res, tokosun_equal_size=t_res)
         print(json.dumps(out))
         return
     if gup:  # the new design beside the tier's closest model at equal width and depth

@@ -885,7 +885,12 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
         Linear up, dn;
         up.A = in; up.lda = W; up.B = L.up; up.ldb = W; up.C = g->u; up.ldc = F; up.M = M; up.N = F; up.K = W; up.act = poly ? ACT_NONE : ACT_RELU2;
         ZG_TRY(launch_linear(up, f32, s));
-        if (poly) ZG_TRY(launch_polynorm(g->u, F, F, M, L.poly, eps, s));
+        if (poly && M <= kPolyMaxRows) {  // decode steps: the activation where the second product reads its rows
+            dn.a_poly = L.poly;
+            dn.poly_eps = eps;
+        } else if (poly) {
+            ZG_TRY(launch_polynorm(g->u, F, F, M, L.poly, eps, s));
+        }
         dn.A = g->u; dn.lda = F; dn.B = L.down; dn.ldb = F; dn.C = out; dn.ldc = W; dn.M = M; dn.N = W; dn.K = F;
         return launch_linear(dn, f32, s);
     };

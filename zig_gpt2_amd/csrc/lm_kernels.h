@@ -42,6 +42,8 @@ struct Linear {
     float glu_limit = 0.0f;            // GLU_CLIPPED
     const float* glu_scale = nullptr;  // GLU_CLIPPED, batched one-row form: factor of batch z's row (null: 1)
     int glu_gate_col = -1;             // >= 0: the activated row is multiplied by sigmoid(A row[glu_gate_col]) (a gate logit behind gate | up)
+    const float* a_poly = nullptr;     // != null (at most kPolyMaxRows rows): A rows enter as a N(z) + b N(z^2) + c N(z^3) + e, N over the row's K values
+    float poly_eps = 0.0f;
     int nz = 1;
     long long a_zoff = 0, b_zoff = 0, c_zoff = 0;
     const int* z_group = nullptr;
@@ -51,6 +53,7 @@ struct Linear {
 // Picks the row-vector kernel (few rows: decode) or the tiled matrix-core kernel (prompt portions).
 int launch_linear(const Linear& L, bool f32, hipStream_t s);
 constexpr int kGemvMaxRows = 8;
+constexpr int kPolyMaxRows = 2;
 // Two products of one-row batches (M == 1 each) in ONE launch of the row-vector kernel; whatever does not fit that form runs as two
 // launches.  Neither product may read what the other writes.
 int launch_linear_pair(const Linear& a, const Linear& b, bool f32, hipStream_t s);

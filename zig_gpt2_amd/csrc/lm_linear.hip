@@ -41,6 +41,8 @@ struct LinArgs {
     float glu_limit;
     const float* glu_scale;
     int glu_gate_col;
+    const float* a_poly;
+    float poly_eps;
     int a_vec, b_vec;  // 16-byte loads allowed (alignment of base, leading dimension and batch offsets)
 };
 
@@ -92,7 +94,43 @@ __device__ __forceinline__ f32x4 load_a4(const float* a, int k, int K, bool vec)
 }
 
 // ------------------------------------------------------------------------------------------------ few rows
-template <int MR>
+// Rows that enter through the polynomial a N(z) + b N(z^2) + c N(z^3) + e (N divides the row by its root mean square): the statistics
+// are sums over the same row, so one pass gathers them beside the products with z, z^2, z^3 and 1, and they meet at the end.
+struct PolySums {
+    float q1 = 0.0f, q2 = 0.0f, q3 = 0.0f;  // sums of z^2, z^4, z^6
+    float d0[4] = {0.0f, 0.0f, 0.0f, 0.0f}, d1[4] = {0.0f, 0.0f, 0.0f, 0.0f};  // the two weight rows with z, z^2, z^3, 1
+    __device__ __forceinline__ void add(float z, float w0, float w1) {
+        const float q = z * z, c = q * z;
+        q1 += q;
+        q2 = fmaf(q, q, q2);
+        q3 = fmaf(c, c, q3);
+        d0[0] = fmaf(z, w0, d0[0]); d1[0] = fmaf(z, w1, d1[0]);
+        d0[1] = fmaf(q, w0, d0[1]); d1[1] = fmaf(q, w1, d1[1]);
+        d0[2] = fmaf(c, w0, d0[2]); d1[2] = fmaf(c, w1, d1[2]);
+        d0[3] += w0; d1[3] += w1;
+    }
+    __device__ __forceinline__ void add8(const f32x4& a0, const f32x4& a1, const float* w0, const float* w1) {
+        add(a0.x, w0[0], w1[0]); add(a0.y, w0[1], w1[1]); add(a0.z, w0[2], w1[2]); add(a0.w, w0[3], w1[3]);
+        add(a1.x, w0[4], w1[4]); add(a1.y, w0[5], w1[5]); add(a1.z, w0[6], w1[6]); add(a1.w, w0[7], w1[7]);
+    }
+    __device__ __forceinline__ void reduce_wave() {
+        q1 = wave_allsum(q1);
+        q2 = wave_allsum(q2);
+        q3 = wave_allsum(q3);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            d0[i] = wave_allsum(d0[i]);
+            d1[i] = wave_allsum(d1[i]);
+        }
+    }
+};
+__device__ __forceinline__ float poly_value(const LinArgs& p, float q1, float q2, float q3, const float* d) {
+    const float K = (float)p.K, eps = p.poly_eps;
+    return (p.a_poly[0] / sqrtf(q1 / K + eps) * d[0] + p.a_poly[1] / sqrtf(q2 / K + eps) * d[1]) +
+           (p.a_poly[2] / sqrtf(q3 / K + eps) * d[2] + p.a_poly[3] * d[3]);
+}
+
+template <int MR, bool POLY = false>
 __device__ __forceinline__ void gemv_body(const LinArgs& p, const int z) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n0 = blockIdx.x * 8 + wave * 2;
@@ -120,6 +158,7 @@ __device__ __forceinline__ void gemv_body(const LinArgs& p, const int z) {
     float acc0[MR], acc1[MR];
 #pragma unroll
     for (int m = 0; m < MR; ++m) acc0[m] = acc1[m] = 0.0f;
+    PolySums ps[POLY ? MR : 1];
     // two K pieces per trip, all four weight vectors requested before the first is used: rows of up to 1024 columns cost one
     // memory round trip
     constexpr int U = MR <= 2 ? 2 : 1;
@@ -148,6 +187,11 @@ __device__ __forceinline__ void gemv_body(const LinArgs& p, const int z) {
                 av[u][0] = a0;
                 av[u][1] = a1;
             }
+            if constexpr (POLY) {
+#pragma unroll
+                for (int u = 0; u < U; ++u) ps[m].add8(av[u][0], av[u][1], wa[u], wb[u]);
+                continue;
+            }
             float s0 = acc0[m], s1 = acc1[m];
 #pragma unroll
             for (int u = 0; u < U; ++u) {
@@ -167,7 +211,12 @@ __device__ __forceinline__ void gemv_body(const LinArgs& p, const int z) {
     }
 #pragma unroll
     for (int m = 0; m < MR; ++m) {
-        const float s0 = wave_allsum(acc0[m]), s1 = wave_allsum(acc1[m]);
+        if constexpr (POLY) {
+            ps[m].reduce_wave();
+            acc0[m] = poly_value(p, ps[m].q1, ps[m].q2, ps[m].q3, ps[m].d0);
+            acc1[m] = poly_value(p, ps[m].q1, ps[m].q2, ps[m].q3, ps[m].d1);
+        }
+        const float s0 = POLY ? acc0[m] : wave_allsum(acc0[m]), s1 = POLY ? acc1[m] : wave_allsum(acc1[m]);
         if (lane == 0 && m < p.M) {
             C[(long long)m * p.ldc + n0] = apply_act(s0, p);
             if (two) C[(long long)m * p.ldc + n0 + 1] = apply_act(s1, p);
@@ -175,9 +224,9 @@ __device__ __forceinline__ void gemv_body(const LinArgs& p, const int z) {
     }
 }
 
-template <int MR>
+template <int MR, bool POLY>
 __global__ __launch_bounds__(256) void lm_gemv_kernel(const LinArgs p) {
-    gemv_body<MR>(p, blockIdx.z);
+    gemv_body<MR, POLY>(p, blockIdx.z);
 }
 
 // Two products of one-row batches in one launch: batches [0, nz_a) are product a's, the rest product b's (the chosen experts and the
@@ -191,9 +240,9 @@ __global__ __launch_bounds__(256) void lm_gemv_pair_kernel(const LinArgs a, cons
 // a few MB is requested whole in one go by thousands of waves instead of trip by trip by a few hundred (a 1600 x 1600 matrix:
 // 800 workgroups, every 16-byte piece in flight at once); the quarter sums meet in the LDS.  The summation order of an output
 // depends on K alone.
-template <int MR>
+template <int MR, bool POLY>
 __global__ __launch_bounds__(256) void lm_gemv_ks_kernel(const LinArgs p) {
-    __shared__ float s_part[4][MR][2];
+    __shared__ float s_part[4][MR][POLY ? 11 : 2];
     const int z = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n0 = blockIdx.x * 2;
     const bf16_t* B = p.B + (long long)(p.z_group ? p.z_group[z] : z) * p.b_zoff;
@@ -218,6 +267,7 @@ __global__ __launch_bounds__(256) void lm_gemv_ks_kernel(const LinArgs p) {
     float acc0[MR], acc1[MR];
 #pragma unroll
     for (int m = 0; m < MR; ++m) acc0[m] = acc1[m] = 0.0f;
+    PolySums ps[POLY ? MR : 1];
     const int kq = (((p.K + 3) / 4) + 7) & ~7;  // a wave's quarter of K, a multiple of 8
     const int k_lo = wave * kq, k_hi = min(p.K, k_lo + kq);
     constexpr int U = 2;
@@ -243,6 +293,10 @@ __global__ __launch_bounds__(256) void lm_gemv_ks_kernel(const LinArgs p) {
                     a1.x = glu_on_load(a1.x, u1.x, p, asc[m]) * agate[m]; a1.y = glu_on_load(a1.y, u1.y, p, asc[m]) * agate[m];
                     a1.z = glu_on_load(a1.z, u1.z, p, asc[m]) * agate[m]; a1.w = glu_on_load(a1.w, u1.w, p, asc[m]) * agate[m];
                 }
+                if constexpr (POLY) {
+                    ps[m].add8(a0, a1, wa[u], wb[u]);
+                    continue;
+                }
                 s0 = fmaf(a0.x, wa[u][0], s0); s1 = fmaf(a0.x, wb[u][0], s1);
                 s0 = fmaf(a0.y, wa[u][1], s0); s1 = fmaf(a0.y, wb[u][1], s1);
                 s0 = fmaf(a0.z, wa[u][2], s0); s1 = fmaf(a0.z, wb[u][2], s1);
@@ -255,6 +309,29 @@ __global__ __launch_bounds__(256) void lm_gemv_ks_kernel(const LinArgs p) {
             acc0[m] = s0;
             acc1[m] = s1;
         }
+    }
+    if constexpr (POLY) {
+#pragma unroll
+        for (int m = 0; m < MR; ++m) {
+            ps[m].reduce_wave();
+            if (lane == 0) {
+                float* o = s_part[wave][m];
+                o[0] = ps[m].q1; o[1] = ps[m].q2; o[2] = ps[m].q3;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    o[3 + i] = ps[m].d0[i];
+                    o[7 + i] = ps[m].d1[i];
+                }
+            }
+        }
+        __syncthreads();
+        if (threadIdx.x < MR * 2) {
+            const int m = threadIdx.x >> 1, c = threadIdx.x & 1;
+            auto sum4 = [&](int i) { return (s_part[0][m][i] + s_part[1][m][i]) + (s_part[2][m][i] + s_part[3][m][i]); };
+            const float d[4] = {sum4(3 + 4 * c), sum4(4 + 4 * c), sum4(5 + 4 * c), sum4(6 + 4 * c)};
+            if (m < p.M && n0 + c < p.N) C[(long long)m * p.ldc + n0 + c] = apply_act(poly_value(p, sum4(0), sum4(1), sum4(2), d), p);
+        }
+        return;
     }
 #pragma unroll
     for (int m = 0; m < MR; ++m) {
@@ -484,6 +561,8 @@ LinArgs make_args(const Linear& L) {
     p.a_div = L.a_div; p.act = L.act; p.n_groups = L.grp_off ? L.n_groups : 0; p.a_glu = L.a_glu;
     p.act_a = L.act_a; p.act_b = L.act_b; p.glu_kind = L.glu_kind; p.glu_limit = L.glu_limit; p.glu_scale = L.glu_scale;
     p.glu_gate_col = L.glu_gate_col;
+    p.a_poly = L.a_poly;
+    p.poly_eps = L.poly_eps;
     p.a_vec = ((reinterpret_cast<uintptr_t>(L.A) & 15) == 0 && L.lda % 4 == 0 && L.a_zoff % 4 == 0) ? 1 : 0;
     p.b_vec = ((reinterpret_cast<uintptr_t>(L.B) & 15) == 0 && L.ldb % 8 == 0 && L.b_zoff % 8 == 0) ? 1 : 0;
     return p;
@@ -494,21 +573,28 @@ int launch_linear(const Linear& L, bool f32, hipStream_t s) {
     if (L.M <= 0 || L.N <= 0 || L.nz <= 0) return ZG_OK;
     ZG_REQUIRE(L.K > 0 && L.A && L.B && L.C, ZG_ERR_ARG, "linear: empty operand");
     ZG_REQUIRE(L.a_div >= 1, ZG_ERR_ARG, "linear: a_div %d", L.a_div);
+    ZG_REQUIRE(!L.a_poly || (L.M <= kPolyMaxRows && L.a_glu == 0 && !L.grp_off), ZG_ERR_ARG, "linear: the polynomial activation on load is for %d rows at most",
+               kPolyMaxRows);
     const LinArgs p = make_args(L);
     if (!L.grp_off && L.M <= kGemvMaxRows) {
         if (takes_k_split(L)) {  // long rows, one or two of them, few batches: K split over the waves, two weight rows per workgroup
             const dim3 gks((L.N + 1) / 2, 1, L.nz);  // (from four rows on the activations are re-read by too many workgroups: measured slower)
-            if (L.M == 1) lm_gemv_ks_kernel<1><<<gks, 256, 0, s>>>(p);
-            else lm_gemv_ks_kernel<2><<<gks, 256, 0, s>>>(p);
+            if (L.a_poly) {
+                if (L.M == 1) lm_gemv_ks_kernel<1, true><<<gks, 256, 0, s>>>(p);
+                else lm_gemv_ks_kernel<2, true><<<gks, 256, 0, s>>>(p);
+            } else if (L.M == 1) lm_gemv_ks_kernel<1, false><<<gks, 256, 0, s>>>(p);
+            else lm_gemv_ks_kernel<2, false><<<gks, 256, 0, s>>>(p);
             note_kernel("lm_gemv_ks_kernel<%d>", L.M);
             ZG_HIP(hipGetLastError());
             return ZG_OK;
         }
         const dim3 grid((L.N + 7) / 8, 1, L.nz);
-        if (L.M == 1) lm_gemv_kernel<1><<<grid, 256, 0, s>>>(p);
-        else if (L.M == 2) lm_gemv_kernel<2><<<grid, 256, 0, s>>>(p);
-        else if (L.M <= 4) lm_gemv_kernel<4><<<grid, 256, 0, s>>>(p);
-        else lm_gemv_kernel<8><<<grid, 256, 0, s>>>(p);
+        if (L.a_poly && L.M == 1) lm_gemv_kernel<1, true><<<grid, 256, 0, s>>>(p);
+        else if (L.a_poly) lm_gemv_kernel<2, true><<<grid, 256, 0, s>>>(p);
+        else if (L.M == 1) lm_gemv_kernel<1, false><<<grid, 256, 0, s>>>(p);
+        else if (L.M == 2) lm_gemv_kernel<2, false><<<grid, 256, 0, s>>>(p);
+        else if (L.M <= 4) lm_gemv_kernel<4, false><<<grid, 256, 0, s>>>(p);
+        else lm_gemv_kernel<8, false><<<grid, 256, 0, s>>>(p);
         note_kernel("lm_gemv_kernel<%d>", L.M == 1 ? 1 : L.M == 2 ? 2 : L.M <= 4 ? 4 : 8);
         ZG_HIP(hipGetLastError());
         return ZG_OK;

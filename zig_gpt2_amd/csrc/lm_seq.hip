@@ -74,6 +74,52 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const float* in, int l
     }
 }
 
+// Steps of many rows, short convolutions: a thread takes kConvRows consecutive rows of a channel, so weights and inputs are read
+// once and the window slides through registers; a row that opens an entry refills the window from its slot's tail.  Sums in the order
+// of the kernel above.
+constexpr int kConvRows = 8;
+template <int TAPS>
+__global__ __launch_bounds__(256) void causal_conv_rows_kernel(const float* in, int ld_in, float* out, int ld_out, int C, int M, const float* w,
+                                                               const float* bias, const float* pre_bias, int flags, const float* tail,
+                                                               size_t slot_stride, const int* row_off, const int* row_slot) {
+    constexpr int K = TAPS - 1;
+    const int m0 = blockIdx.x * kConvRows, c = blockIdx.y * blockDim.x + threadIdx.x;
+    if (c >= C) return;
+    const float pb = pre_bias ? pre_bias[c] : 0.0f, b0 = bias ? bias[c] : 0.0f;
+    float wt[TAPS], cur[kConvRows], win[TAPS];  // win: the K inputs in front of the row, oldest first, then the row's own
+    int off[kConvRows];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wt[j] = w[(size_t)c * TAPS + j];
+#pragma unroll
+    for (int i = 0; i < kConvRows; ++i) {
+        const int m = min(m0 + i, M - 1);
+        cur[i] = in[(size_t)m * ld_in + c] + pb;
+        off[i] = row_off[m];
+    }
+#pragma unroll
+    for (int j = 0; j < K; ++j) {  // in front of the first row: rows of the same entry, or the tail
+        const int src = off[0] - K + j;
+        win[j] = src >= 0 ? in[(size_t)(m0 - K + j) * ld_in + c] + pb : tail[(size_t)row_slot[m0] * slot_stride + (size_t)(K + src) * C + c];
+    }
+#pragma unroll
+    for (int i = 0; i < kConvRows; ++i) {
+        if (i > 0 && off[i] == 0) {
+            const float* tl = tail + (size_t)row_slot[min(m0 + i, M - 1)] * slot_stride + c;
+#pragma unroll
+            for (int j = 0; j < K; ++j) win[j] = tl[(size_t)j * C];
+        }
+        win[K] = cur[i];
+        float acc = b0;
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) acc = fmaf(wt[j], win[j], acc);
+        if (flags & CONV_RESIDUAL) acc += cur[i];
+        if (flags & CONV_SILU) acc = silu_f(acc);
+        if (m0 + i < M) out[(size_t)(m0 + i) * ld_out + c] = acc;
+#pragma unroll
+        for (int j = 0; j < K; ++j) win[j] = win[j + 1];
+    }
+}
+
 // The new tail of every entry's slot: the last taps - 1 of (old tail, the entry's inputs).  A thread reads all it needs
 // before it writes, and no other thread touches its channel of its slot.
 __global__ __launch_bounds__(256) void conv_tail_kernel(const float* in, int ld_in, int C, int taps, const float* pre_bias, float* tail,
@@ -1252,10 +1298,19 @@ int launch_causal_conv(const ConvArgs& a, int M, int n_entries, bool one_row_eac
     ZG_REQUIRE(a.taps >= 1 && a.taps <= kMaxTaps, ZG_ERR_UNSUPPORTED, "convolution: %d taps (1 to %d)", a.taps, kMaxTaps);
     ZG_REQUIRE(a.in != a.out, ZG_ERR_ARG, "convolution: in place");
     const int bx = a.C >= 256 ? 256 : 64;
-    causal_conv_kernel<<<dim3(M, (a.C + bx - 1) / bx), bx, 0, s>>>(a.in, a.ld_in, a.out, a.ld_out, a.C, a.taps, a.w, a.bias, a.pre_bias, a.flags, a.tail,
+    const dim3 rgrid((M + kConvRows - 1) / kConvRows, (a.C + bx - 1) / bx);
+#define ZG_CONV_ROWS(T_)                                                                                                                          \
+    causal_conv_rows_kernel<T_><<<rgrid, bx, 0, s>>>(a.in, a.ld_in, a.out, a.ld_out, a.C, M, a.w, a.bias, a.pre_bias, a.flags, a.tail, a.slot_stride, row_off, \
+                                                     row_slot)
+    const bool rows = M > kGemvMaxRows;
+    if (rows && a.taps == 2) ZG_CONV_ROWS(2);
+    else if (rows && a.taps == 3) ZG_CONV_ROWS(3);
+    else if (rows && a.taps == 4) ZG_CONV_ROWS(4);
+    else causal_conv_kernel<<<dim3(M, (a.C + bx - 1) / bx), bx, 0, s>>>(a.in, a.ld_in, a.out, a.ld_out, a.C, a.taps, a.w, a.bias, a.pre_bias, a.flags, a.tail,
                                                                  a.slot_stride, row_off, row_slot, one_row_each ? 1 : 0);
+#undef ZG_CONV_ROWS
     ZG_HIP(hipGetLastError());
-    if (a.taps > 1 && !one_row_each) {
+    if (a.taps > 1 && !(one_row_each && !rows)) {
         conv_tail_kernel<<<dim3(n_entries, (a.C + bx - 1) / bx), bx, 0, s>>>(a.in, a.ld_in, a.C, a.taps, a.pre_bias, a.tail, a.slot_stride, ent_start,
                                                                            ent_len, ent_slot);
         ZG_HIP(hipGetLastError());
@@ -1330,8 +1385,10 @@ int launch_head_norm_prep(float* qk, int ld, int M, int H, int G, int D, float e
 }
 
 size_t window_split_workspace(int rows, int H, int V, int key_capacity, int* n_split_out) {
-    // shares of kMixTile keys: up to kWinSplits of them for steps of few rows (many workgroups per row), up to 16 for portions
-    const int n_split = std::max(1, std::min(rows <= kGemvMaxRows ? kWinSplits : 16, (key_capacity + kMixTile - 1) / kMixTile));
+    // shares of kMixTile keys: up to kWinSplits of them for steps of few rows (many workgroups per row); portions: up to 16, fewer where
+    // the rows alone (32 of them to a workgroup) fill the chip — every share is one more partial sum to write and to add
+    const int most = rows <= kGemvMaxRows ? kWinSplits : std::max(4, std::min(16, 1024 / ((rows + 31) / 32)));
+    const int n_split = std::max(1, std::min(most, (key_capacity + kMixTile - 1) / kMixTile));
     if (n_split_out) *n_split_out = n_split;
     return (size_t)rows * H * key_capacity + (size_t)rows * n_split * H * 2 + (size_t)rows * n_split * H * V;
 }

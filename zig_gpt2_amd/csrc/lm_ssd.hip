@@ -40,6 +40,7 @@ constexpr int kSsdCols = 32;
 constexpr int kSsdGroups = 8;
 constexpr int kSsdBlock = 8;
 constexpr int kSsdTaps = 16;
+constexpr int kSsdFastTaps = 4;
 
 template <int R, bool CONV>
 __global__ __launch_bounds__(256) void ssd_scan_kernel(const SsdArgs a, const ConvArgs cv, const int* ent_start, const int* ent_len, const int* ent_slot) {
@@ -76,9 +77,18 @@ __global__ __launch_bounds__(256) void ssd_scan_kernel(const SsdArgs a, const Co
                     const float* tl = cv.tail + (size_t)slot * cv.slot_stride;
                     const int K = cv.taps - 1;
                     float acc = cv.bias ? cv.bias[ch] : 0.0f;
+                    if (cv.taps <= kSsdFastTaps) {  // weights and tail requested together
+                        float wt[kSsdFastTaps], tv[kSsdFastTaps];
 #pragma unroll
-                    for (int j = 0; j < kSsdTaps; ++j)
-                        if (j < cv.taps) acc = fmaf(cv.w[(size_t)ch * cv.taps + j], j < K ? tl[(size_t)j * cv.C + ch] : v, acc);
+                        for (int j = 0; j < kSsdFastTaps; ++j) {
+                            wt[j] = cv.w[(size_t)ch * cv.taps + min(j, K)];
+                            tv[j] = K > 0 ? tl[(size_t)min(j, K - 1) * cv.C + ch] : 0.0f;
+                        }
+#pragma unroll
+                        for (int j = 0; j < kSsdFastTaps; ++j) acc = j <= K ? fmaf(wt[j], j < K ? tv[j] : v, acc) : acc;
+                    } else {
+                        for (int j = 0; j < cv.taps; ++j) acc = fmaf(cv.w[(size_t)ch * cv.taps + j], j < K ? tl[(size_t)j * cv.C + ch] : v, acc);
+                    }
                     v = silu_f(acc);
                 }
             }
@@ -125,7 +135,8 @@ __global__ __launch_bounds__(256) void ssd_scan_kernel(const SsdArgs a, const Co
 // v_mfma_f32_32x32x2_f32); l_t = -exp(a_log) dt_t, L(j, i) = exp(l_(j+1) + ... + l_i):
 //   state   E = sum_j L(j, n-1) dt_j B_j x_j^T                      the chunk's end state from zero          (per chunk)
 //   carry   S_start(c + 1) = L(-1, n-1) S_start(c) + E_c            down the chunks of an entry              (launch_state_carry)
-//   output  y_i = sum_(j<=i) L(j, i) dt_j (C_i . B_j) x_j + L(-1, i) S_start^T C_i + skip x_i, times silu(z)  (per chunk)
+//   output  y_i = sum_(j<=i) L(j, i) dt_j (C_i . B_j) x_j + L(-1, i) S_start^T C_i + skip x_i, times silu(z)  (per chunk; the skip
+//           factor rides on the diagonal of the first sum's weights)
 // The logarithms inside a chunk are added up directly between j and i (all of one sign: nothing cancels, and a token that forgets
 // everything does not blur the decays behind it).
 constexpr int kSsdChunk = 32;
@@ -150,6 +161,21 @@ __global__ __launch_bounds__(256) void ssd_chunk_state_kernel(const SsdArgs a, c
     const int h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 31, kh = lane >> 5;
     const int n = min(kSsdChunk, ent_len[e] - c * kSsdChunk), m0 = ent_start[e] + c * kSsdChunk;
     const int HV = a.H * a.V, grp = h / (a.H / a.G);
+    const float* base = a.xbc + (size_t)m0 * a.ld_xbc;
+    float* E = wsB + ((size_t)blockIdx.x * a.H + h) * a.N * a.V;
+    const int tilesN = (a.N + 31) / 32, tilesV = (a.V + 31) / 32;
+    float av[16], bv[16];
+    auto fetch = [&](int tile) {  // the token is the inner dimension (tokens beyond the chunk's end weigh nothing)
+        const int ob = HV + grp * a.N + min((tile / tilesV) * 32 + r, a.N - 1), ox = h * a.V + min((tile % tilesV) * 32 + r, a.V - 1);
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            const float* row = base + min(kh * 16 + t, n - 1) * a.ld_xbc;
+            av[t] = row[ob];
+            bv[t] = row[ox];
+        }
+    };
+    int tile = blockIdx.z * 4 + wave;
+    if (tile < tilesN * tilesV) fetch(tile);  // in flight beside the step sizes
     float dt = 0.0f;
     if (threadIdx.x < kSsdChunk) {
         const int t = threadIdx.x;
@@ -164,19 +190,9 @@ __global__ __launch_bounds__(256) void ssd_chunk_state_kernel(const SsdArgs a, c
         if (threadIdx.x == 0 && blockIdx.z == 0) wsA[(size_t)blockIdx.x * a.H + h] = expf(run + s_l[0]);
     }
     __syncthreads();
-    const float* bbase = a.xbc + (size_t)m0 * a.ld_xbc + HV + (size_t)grp * a.N;
-    const float* xbase = a.xbc + (size_t)m0 * a.ld_xbc + (size_t)h * a.V;
-    float* E = wsB + ((size_t)blockIdx.x * a.H + h) * a.N * a.V;
-    const int tilesN = (a.N + 31) / 32, tilesV = (a.V + 31) / 32;
-    for (int tile = blockIdx.z * 4 + wave; tile < tilesN * tilesV; tile += 4 * gridDim.z) {
+    for (bool first = true; tile < tilesN * tilesV; tile += 4 * gridDim.z, first = false) {
         const int i0 = (tile / tilesV) * 32, v0 = (tile % tilesV) * 32;
-        float av[16], bv[16];
-#pragma unroll
-        for (int t = 0; t < 16; ++t) {  // the token is the inner dimension
-            const int j = kh * 16 + t;
-            av[t] = (j < n && i0 + r < a.N) ? bbase[(size_t)j * a.ld_xbc + i0 + r] : 0.0f;
-            bv[t] = (j < n && v0 + r < a.V) ? xbase[(size_t)j * a.ld_xbc + v0 + r] : 0.0f;
-        }
+        if (!first) fetch(tile);
         f32x16_ssd acc;
 #pragma unroll
         for (int i = 0; i < 16; ++i) acc[i] = 0.0f;
@@ -195,7 +211,7 @@ __global__ __launch_bounds__(256) void ssd_chunk_state_kernel(const SsdArgs a, c
 // state channels (eight at a time), their shares meet in the LDS; then a wave owns (head, 32 value columns) units.
 constexpr int kSsdHeads = 4;  // most heads of a workgroup
 
-__global__ __launch_bounds__(256) void ssd_chunk_out_kernel(const SsdArgs a, const int* ent_start, const int* ent_len, int n_entries,
+__global__ __launch_bounds__(256, 2) void ssd_chunk_out_kernel(const SsdArgs a, const int* ent_start, const int* ent_len, int n_entries,
                                                             const float* __restrict__ wsB, int hb, int blocks_per_group) {
     extern __shared__ __attribute__((aligned(16))) float s_ssd[];
     __shared__ float s_p[4][32][33];
@@ -206,13 +222,26 @@ __global__ __launch_bounds__(256) void ssd_chunk_out_kernel(const SsdArgs a, con
     const int n = min(kSsdChunk, ent_len[e] - c * kSsdChunk), m0 = ent_start[e] + c * kSsdChunk;
     const int grp = blockIdx.y / blocks_per_group, per = a.H / a.G;
     const int hl0 = (blockIdx.y % blocks_per_group) * hb, nh = min(hb, per - hl0), h0 = grp * per + hl0;  // heads [h0, h0 + nh)
-    const int HV = a.H * a.V, N8 = (a.N + 7) / 8, ldC = 8 * N8 + 4;
-    float* s_C = s_ssd;  // [32][ldC], zero beyond N and beyond the chunk
+    const int HV = a.H * a.V, N8 = (a.N + 31) / 32 * 4, ldC = 8 * N8 + 4;  // (groups of eight state channels, a multiple of four of them)
+    float* s_C = s_ssd;  // [32][ldC], zero beyond N (rows beyond the chunk repeat its last one: nothing of them is written)
     const float* brow = a.xbc + (size_t)m0 * a.ld_xbc + HV + (size_t)grp * a.N;
     const float* crow = brow + (size_t)a.G * a.N;
-    for (int idx = tid; idx < 32 * 8 * N8; idx += 256) {
-        const int t = idx / (8 * N8), ch = idx % (8 * N8);
-        s_C[t * ldC + ch] = (t < n && ch < a.N) ? crow[(size_t)t * a.ld_xbc + ch] : 0.0f;
+    const bool vec = a.N % 4 == 0 && a.ld_xbc % 4 == 0 && HV % 4 == 0 && (reinterpret_cast<uintptr_t>(a.xbc) & 15) == 0;
+    // four channels of a row; beyond N whatever is there (the query rows hold zeros beyond N, so it weighs nothing)
+    auto row4 = [&](const float* row, int ch) {
+        if (vec) return *reinterpret_cast<const f32x4*>(row + min(ch, a.N - 4));
+        return f32x4{row[min(ch, a.N - 1)], row[min(ch + 1, a.N - 1)], row[min(ch + 2, a.N - 1)], row[min(ch + 3, a.N - 1)]};
+    };
+    {
+        const int t = tid >> 3;
+        for (int ch = 4 * (tid & 7); ch < 8 * N8; ch += 32) {
+            f32x4 v = row4(crow + (size_t)min(t, n - 1) * a.ld_xbc, ch);
+            v.x = ch + 0 < a.N ? v.x : 0.0f;
+            v.y = ch + 1 < a.N ? v.y : 0.0f;
+            v.z = ch + 2 < a.N ? v.z : 0.0f;
+            v.w = ch + 3 < a.N ? v.w : 0.0f;
+            *reinterpret_cast<f32x4*>(s_C + t * ldC + ch) = v;
+        }
     }
     if (tid < 32 * nh) {
         const int hh = tid >> 5, t = tid & 31;
@@ -231,22 +260,12 @@ __global__ __launch_bounds__(256) void ssd_chunk_out_kernel(const SsdArgs a, con
 #pragma unroll
     for (int i = 0; i < 16; ++i) acc[i] = 0.0f;
     {
-        const bool vec = a.N % 4 == 0 && a.ld_xbc % 4 == 0 && HV % 4 == 0 && (reinterpret_cast<uintptr_t>(a.xbc) & 15) == 0;
         const float* br = brow + (size_t)min(r, n - 1) * a.ld_xbc;
-        for (int g8 = wave; g8 < N8; g8 += 4) {  // channels 8 g8 + 4 half + u of rows r: query row from the LDS, key row from memory
-            const int ch = 8 * g8 + 4 * kh;
-            const f32x4 q = *reinterpret_cast<const f32x4*>(s_C + r * ldC + ch);
-            f32x4 k = {0.0f, 0.0f, 0.0f, 0.0f};
-            if (r < n) {
-                if (vec && ch + 4 <= a.N) {
-                    k = *reinterpret_cast<const f32x4*>(br + ch);
-                } else {
-                    k.x = ch + 0 < a.N ? br[ch + 0] : 0.0f;
-                    k.y = ch + 1 < a.N ? br[ch + 1] : 0.0f;
-                    k.z = ch + 2 < a.N ? br[ch + 2] : 0.0f;
-                    k.w = ch + 3 < a.N ? br[ch + 3] : 0.0f;
-                }
-            }
+        // channels 8 g8 + 4 half + u of rows r: query row from the LDS, key row from memory (requested one group ahead)
+        f32x4 kn = row4(br, 8 * wave + 4 * kh);
+        for (int g8 = wave; g8 < N8; g8 += 4) {
+            const f32x4 k = kn, q = *reinterpret_cast<const f32x4*>(s_C + r * ldC + 8 * g8 + 4 * kh);
+            kn = row4(br, 8 * (g8 + 4) + 4 * kh);
             acc = __builtin_amdgcn_mfma_f32_32x32x2f32(q.x, k.x, acc, 0, 0, 0);
             acc = __builtin_amdgcn_mfma_f32_32x32x2f32(q.y, k.y, acc, 0, 0, 0);
             acc = __builtin_amdgcn_mfma_f32_32x32x2f32(q.z, k.z, acc, 0, 0, 0);
@@ -265,39 +284,56 @@ __global__ __launch_bounds__(256) void ssd_chunk_out_kernel(const SsdArgs a, con
     for (int u = wave; u < nh * tilesV; u += 4) {
         const int hh = u / tilesV, h = h0 + hh, v0 = (u % tilesV) * 32;
         const bool col_ok = v0 + r < a.V;
-        const float* xbase = a.xbc + (size_t)m0 * a.ld_xbc + (size_t)h * a.V + v0 + r;
-        const float* S = wsB + ((size_t)blockIdx.x * a.H + h) * a.N * a.V + v0 + r;  // the chunk's start state (the carry left it here)
+        // (columns beyond V read the last one, tokens beyond the chunk its last: they weigh nothing or are not written)
+        const int col = h * a.V + min(v0 + r, a.V - 1);
+        const float* xbase = a.xbc + (size_t)m0 * a.ld_xbc + col;
+        const float* S = wsB + (size_t)blockIdx.x * a.H * a.N * a.V + (size_t)h * a.N * a.V + min(v0 + r, a.V - 1);  // the chunk's start state (the carry left it here)
         float xv[16];
 #pragma unroll
-        for (int t = 0; t < 16; ++t) {
-            const int j = kh * 16 + t;
-            xv[t] = (j < n && col_ok) ? xbase[(size_t)j * a.ld_xbc] : 0.0f;
+        for (int t = 0; t < 16; ++t) xv[t] = xbase[min(kh * 16 + t, n - 1) * a.ld_xbc];
+        float* obase = a.out + (size_t)m0 * a.ldo + col;
+        const float* zbase = a.z + (size_t)m0 * a.ld_proj + col;
+        float zv[16];  // the gates of the outputs this lane will write
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const int qi = 8 * (i >> 2) + 4 * kh + (i & 3);
+            zv[i] = zbase[min(qi, n - 1) * a.ld_proj];
         }
-        // the start state's share
+        // the start state's share, 16 state rows requested while the 16 before are multiplied
         f32x16_ssd accS;
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
             acc[i] = 0.0f;
             accS[i] = 0.0f;
         }
-        for (int g0 = 0; g0 < N8; g0 += 4) {  // 16 state rows requested at a time
-            float sv[16];
+        float sv[2][8];
+        auto state_rows = [&](int g0, float* dst) {
 #pragma unroll
-            for (int t = 0; t < 16; ++t) {
+            for (int t = 0; t < 8; ++t) {
                 const int ch = 8 * (g0 + (t >> 2)) + 4 * kh + (t & 3);
-                sv[t] = (ch < a.N && col_ok) ? S[(size_t)ch * a.V] : 0.0f;
+                dst[t] = S[min(ch, a.N - 1) * a.V];
             }
+        };
+        auto state_product = [&](int g0, const float* src) {
 #pragma unroll
-            for (int t4 = 0; t4 < 4; ++t4) {
-                const f32x4 q = *reinterpret_cast<const f32x4*>(s_C + r * ldC + min(8 * (g0 + t4), 8 * (N8 - 1)) + 4 * kh);
-                accS = __builtin_amdgcn_mfma_f32_32x32x2f32(q.x, sv[4 * t4 + 0], accS, 0, 0, 0);
-                accS = __builtin_amdgcn_mfma_f32_32x32x2f32(q.y, sv[4 * t4 + 1], accS, 0, 0, 0);
-                accS = __builtin_amdgcn_mfma_f32_32x32x2f32(q.z, sv[4 * t4 + 2], accS, 0, 0, 0);
-                accS = __builtin_amdgcn_mfma_f32_32x32x2f32(q.w, sv[4 * t4 + 3], accS, 0, 0, 0);
+            for (int t4 = 0; t4 < 2; ++t4) {
+                const f32x4 q = *reinterpret_cast<const f32x4*>(s_C + r * ldC + 8 * (g0 + t4) + 4 * kh);
+                accS = __builtin_amdgcn_mfma_f32_32x32x2f32(q.x, src[4 * t4 + 0], accS, 0, 0, 0);
+                accS = __builtin_amdgcn_mfma_f32_32x32x2f32(q.y, src[4 * t4 + 1], accS, 0, 0, 0);
+                accS = __builtin_amdgcn_mfma_f32_32x32x2f32(q.z, src[4 * t4 + 2], accS, 0, 0, 0);
+                accS = __builtin_amdgcn_mfma_f32_32x32x2f32(q.w, src[4 * t4 + 3], accS, 0, 0, 0);
             }
+        };
+        state_rows(0, sv[0]);
+        for (int g0 = 0; g0 < N8; g0 += 4) {
+            state_rows(g0 + 2, sv[1]);
+            state_product(g0, sv[0]);
+            if (g0 + 4 < N8) state_rows(g0 + 4, sv[0]);
+            state_product(g0 + 2, sv[1]);
         }
         // the chunk's own tokens: lane (r, half) weighs the keys half * 16 .. + 15 for query row r, from the nearest back
         float wv[16], run = 0.0f;
+        const float skip = a.skip[h];
         if (kh == 0)
             for (int t = 16; t < 32; ++t) run += t <= r ? s_l[hh][t] : 0.0f;
 #pragma unroll
@@ -305,19 +341,14 @@ __global__ __launch_bounds__(256) void ssd_chunk_out_kernel(const SsdArgs a, con
             const int j = kh * 16 + t;
             if (t < 15 && j < r) run += s_l[hh][j + 1];
             if (t == 15 && kh == 1) run = 0.0f;
-            wv[t] = j <= r ? s_p[0][r][j] * expf(run) * s_dt[hh][j] : 0.0f;
+            wv[t] = j <= r ? s_p[0][r][j] * expf(run) * s_dt[hh][j] + (j == r ? skip : 0.0f) : 0.0f;
         }
 #pragma unroll
         for (int t = 0; t < 16; ++t) acc = __builtin_amdgcn_mfma_f32_32x32x2f32(wv[t], xv[t], acc, 0, 0, 0);
-        const float skip = a.skip[h];
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
             const int qi = 8 * (i >> 2) + 4 * kh + (i & 3);
-            if (qi < n && col_ok) {
-                const size_t m = m0 + qi;
-                const float y = acc[i] + s_pre[hh][qi] * accS[i] + skip * xbase[(size_t)qi * a.ld_xbc];
-                a.out[m * a.ldo + (size_t)h * a.V + v0 + r] = y * silu_f(a.z[m * a.ld_proj + (size_t)h * a.V + v0 + r]);
-            }
+            if (qi < n && col_ok) obase[qi * a.ldo] = (acc[i] + s_pre[hh][qi] * accS[i]) * silu_f(zv[i]);
         }
     }
 }
@@ -325,24 +356,23 @@ __global__ __launch_bounds__(256) void ssd_chunk_out_kernel(const SsdArgs a, con
 // ------------------------------------------------------------------------------------------------ norm in parts, polynomial activation
 constexpr int kPartRegs = 16;  // parts of up to 256 * kPartRegs channels stay in registers
 
-__global__ __launch_bounds__(256) void part_norm_kernel(float* v, int ld, int width, int parts, const float* w, float eps, const ConvArgs cv, int move_tail,
-                                                        const int* row_slot) {
+__global__ __launch_bounds__(256) void part_norm_kernel(float* v, int ld, int width, int parts, const float* w, float eps, const ConvArgs cv, const int* row_slot) {
     __shared__ float s_red[8];
     const int m = blockIdx.x, part = blockIdx.y, n = width / parts;
+    if (part >= parts) {  // the row is its entry's only one: the workgroups behind the parts move the convolution's tail on, 256 channels each
+        const int K = cv.taps - 1, c = (part - parts) * 256 + threadIdx.x;
+        if (c >= cv.C) return;
+        float* tl = cv.tail + (size_t)row_slot[m] * cv.slot_stride + c;
+        float val = cv.in[(size_t)m * cv.ld_in + c];  // every entry takes its successor's place, the newest one the current input
+        for (int i = K - 1; i >= 0; --i) {
+            const float old = tl[(size_t)i * cv.C];
+            tl[(size_t)i * cv.C] = val;
+            val = old;
+        }
+        return;
+    }
     float* p = v + (size_t)m * ld + (size_t)part * n;
     const float* wp = w + (size_t)part * n;
-    if (move_tail) {  // the row is its entry's only one: its channels are shared out over the parts' workgroups
-        float* tl = cv.tail + (size_t)row_slot[m] * cv.slot_stride;
-        const int K = cv.taps - 1;
-        for (int c = part * 256 + threadIdx.x; c < cv.C; c += 256 * parts) {
-            float val[kSsdTaps];
-#pragma unroll
-            for (int i = 0; i < kSsdTaps; ++i) val[i] = i + 1 < K ? tl[(size_t)(i + 1) * cv.C + c] : cv.in[(size_t)m * cv.ld_in + c];
-#pragma unroll
-            for (int i = 0; i < kSsdTaps; ++i)
-                if (i < K) tl[(size_t)i * cv.C + c] = val[i];
-        }
-    }
     if (n <= 256 * kPartRegs) {
         float x[kPartRegs], wr[kPartRegs], ss = 0.0f;
 #pragma unroll
@@ -442,7 +472,7 @@ int launch_ssd_scan(const SsdArgs& a, const ConvArgs* conv, int M, const int* en
         ZG_HIP(hipGetLastError());
         ZG_TRY(launch_state_carry(a.state, a.slot_stride, ent_len, ent_slot, n_entries, a.H, a.N, a.V, cB, cA, 1, kSsdChunk, s));
         const int tilesV = (a.V + 31) / 32, per = a.H / a.G, hb = std::max(1, std::min(std::min(kSsdHeads, per), 4 / tilesV)), bpg = (per + hb - 1) / hb;
-        const size_t lds = (size_t)32 * (8 * ((a.N + 7) / 8) + 4) * sizeof(float);
+        const size_t lds = (size_t)32 * ((a.N + 31) / 32 * 32 + 4) * sizeof(float);
         ssd_chunk_out_kernel<<<dim3(n_chunks, a.G * bpg), 256, lds, s>>>(a, ent_start, ent_len, n_entries, cB, hb, bpg);
         ZG_HIP(hipGetLastError());
         return ZG_OK;
@@ -469,7 +499,8 @@ int launch_part_norm(float* v, int ld, int width, int parts, int M, const float*
     if (M <= 0 || width <= 0) return ZG_OK;
     ZG_REQUIRE(parts >= 1 && parts <= 65535 && width % parts == 0, ZG_ERR_ARG, "norm in parts: %d channels in %d parts", width, parts);
     ZG_REQUIRE(!conv || (conv->taps >= 1 && conv->taps <= kSsdTaps), ZG_ERR_ARG, "norm in parts: a convolution of more than %d taps", kSsdTaps);
-    part_norm_kernel<<<dim3(M, parts), 256, 0, s>>>(v, ld, width, parts, w, eps, conv ? *conv : ConvArgs(), conv && conv->taps > 1 ? 1 : 0, row_slot);
+    const int tail_blocks = conv && conv->taps > 1 ? (conv->C + 255) / 256 : 0;
+    part_norm_kernel<<<dim3(M, parts + tail_blocks), 256, 0, s>>>(v, ld, width, parts, w, eps, conv ? *conv : ConvArgs(), row_slot);
     ZG_HIP(hipGetLastError());
     return ZG_OK;
 }

@@ -350,13 +350,13 @@ class LayerSpec:
                       m + "o": (W, H * V)})
         elif self.mixer == "latent_attention":
             R, KR, QR = self.rot_dim, self.kv_rank, self.q_rank
-            t.update({m + "uk": (H * D, KR), m + "uv": (H * V, KR), m + "o": (W, H * V)})
             if QR:
                 t.update({m + "dq": (QR, W), m + "dq.norm": (QR,), m + "uq": (H * (D + R), QR)})
             else:
                 t[m + "q"] = (H * (D + R), W)
             if self.kv_from is None:
                 t.update({m + "dkv": (KR + R, W), m + "dkv.norm": (KR,)})
+            t.update({m + "uk": (H * D, KR), m + "uv": (H * V, KR), m + "o": (W, H * V)})
             if self.head_gate:
                 t[m + "g"] = (H, W)
         elif self.mixer == "rotary_attention":
