@@ -519,7 +519,7 @@ def duvulix_bench_config(width, n_layers, vocab, chunk=512):
     lat = dict(mixer="latent_attention", heads=heads, dim=64, vdim=64, rot_dim=32, kv_rank=256, scale=(64 + 32) ** -0.5, rot_dims=32, rot_base=10000.0,
                head_gate=True, **dense)
     att = dict(mixer="rotary_attention", heads=heads, kv_heads=kv, dim=64, vdim=64, scale=64 ** -0.5, chunk=chunk, rot_dims=64, rot_base=10000.0,
-               rot_scaling={"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}, **dense)
+               rot_scaling={"factor": 8.0, "original": 1024, "fast": 24.0, "slow": 2.0}, **dense)
     layers = [lm.LayerSpec(**[ssm, lat, dict(lat, kv_from=i - 1), att][i % 4]) for i in range(n_layers)]
     return lm.LMConfig(vocab=vocab, width=width, layers=layers, norm_eps=1e-6, architecture="Duvulix")
 

@@ -68,10 +68,10 @@ def test_rotation_on_hand_made_vectors():
     a = (do.rotate(q, [11], rot) * do.rotate(k, [4], rot)).sum()
     assert abs(a - (do.rotate(q, [107], rot) * do.rotate(k, [100], rot)).sum()) < 1e-9
     # the blend: pairs that turn often keep their frequency, slow ones are divided by the factor
-    f, amp = do.rotary_frequencies({"base": 10000.0, "dims": 64, "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}})
-    g = 10000.0 ** (-2.0 * np.arange(32) / 64)
-    assert np.allclose(f[0], g[0]) and np.allclose(f[-1], g[-1] / 4.0) and abs(amp - (0.1 * math.log(4.0) + 1.0)) < 1e-12
-    assert ((f <= g + 1e-15) & (f >= g / 4.0 - 1e-15)).all()
+    f, amp = do.rotary_frequencies({"base": 30000.0, "dims": 64, "scaling": {"factor": 5.0, "original": 700, "fast": 20.0, "slow": 1.5}})
+    g = 30000.0 ** (-2.0 * np.arange(32) / 64)
+    assert np.allclose(f[0], g[0]) and np.allclose(f[-1], g[-1] / 5.0) and abs(amp - (0.1 * math.log(5.0) + 1.0)) < 1e-12
+    assert ((f <= g + 1e-15) & (f >= g / 5.0 - 1e-15)).all()
 
 
 def test_chunks_on_hand_made_positions():

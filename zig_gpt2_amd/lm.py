@@ -184,8 +184,8 @@ class LayerSpec:
                       rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 10000.0)),
                       rot_scaling=dict(rot["scaling"]) if rot.get("scaling") else None)
         elif kind == "ssd":
-            kw = dict(mixer=kind, heads=int(m["heads"]), vdim=int(m["vdim"]), dim=int(m["state"]), kv_heads=int(m.get("groups", 1)), conv=int(m["conv"]),
-                      norm_groups=int(m.get("norm_groups", 1)))
+            kw = dict(mixer=kind, heads=int(m["heads"]), vdim=int(m["vdim"]), dim=int(m["state"]), kv_heads=int(m.get("groups") or 1), conv=int(m["conv"]),
+                      norm_groups=int(m.get("norm_groups") or 1))
         else:
             kw = dict(mixer=kind, heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]))
         kw.update(rot_halves=bool(fixed.get("rot_halves")))
