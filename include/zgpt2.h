@@ -382,7 +382,8 @@ enum {
                                        2^(-8 (h + 1) / heads) (i - j) for head h (dist_bias 0: not) */
     ZG_LM_MIX_ROTARY_ATTENTION = 8, /* causal grouped-query softmax attention with rotary positions on the first rot_dims channels of q
                                        and k (any pairing, scaled frequencies and amplitude allowed); with chunk > 0 a query sees the keys
-                                       of its own chunk of positions [n chunk, (n + 1) chunk) only, with window > 0 those of its window */
+                                       of its own chunk of positions [n chunk, (n + 1) chunk) only, with window > 0 those of its window.
+                                       Options: proj_bias, value_norm, value_mix, sigmoid_weights (see the fields) */
     ZG_LM_MIX_SSD = 9               /* selective state space with a scalar decay per head and token (Mamba-2): in = [z (heads vdim) |
                                        x (heads vdim) | B (kv_heads dim) | C (kv_heads dim) | dt (heads)] rows of one projection; x, B, C
                                        pass a causal convolution of `conv` taps with bias and silu; dt = softplus(dt + dt_bias);
@@ -393,8 +394,9 @@ enum { ZG_LM_FF_NONE = 0, ZG_LM_FF_DENSE = 1 /* down(act(up h)) */, ZG_LM_FF_MOE
 /* Activation of the dense feed-forward (dense_act). */
 enum {
     ZG_LM_DENSE_RELU2 = 0,   /* relu(z)^2 */
-    ZG_LM_DENSE_POLYNORM = 1 /* a N(z) + b N(z^2) + c N(z^3) + e, N(v) = v / sqrt(mean(v^2) + norm_eps) over the row; the fp32 tensor
+    ZG_LM_DENSE_POLYNORM = 1, /* a N(z) + b N(z^2) + c N(z^3) + e, N(v) = v / sqrt(mean(v^2) + norm_eps) over the row; the fp32 tensor
                                 `mlp.act` holds a, b, c, e */
+    ZG_LM_DENSE_GLU_GELU = 2  /* gated: down(gelu(gate h) * up h), the tanh form of gelu (tensors mlp.gate / up / down) */
 };
 /* Activation of an expert (ff_act) and the rule of the router (router) of ZG_LM_FF_MOE. */
 enum {
@@ -407,10 +409,12 @@ enum {
     ZG_LM_ROUTE_TOP_LOGITS = 1,  /* z = router h + bias (`router.b`); the `top` largest z; weights softmax over the chosen z */
     ZG_LM_ROUTE_SIGMOID_INPUT = 2, /* s = sigmoid(router h); the `top` largest; the weight s (not renormalised) multiplies the expert's
                                      INPUT: the sublayer's output is the plain sum of expert(s h) */
-    ZG_LM_ROUTE_SIGMOID_GROUPS = 3 /* s = sigmoid(router h); experts are ranked by r = s + correction.  The expert list is cut into
+    ZG_LM_ROUTE_SIGMOID_GROUPS = 3, /* s = sigmoid(router h); experts are ranked by r = s + correction.  The expert list is cut into
                                      route_groups contiguous blocks of equal size; a block's rank is r of its best expert plus r of
                                      its second best (a block of one: its only r); experts outside the route_keep top-ranked blocks
                                      get r = -inf; the `top` highest r win; weights s / (sum of the winners' s + 1e-20) * route_scale */
+    ZG_LM_ROUTE_SOFTMAX_GROUPS = 4 /* the same with s = softmax(router h) over all router outputs (the pass-through ones of `identity`
+                                     included) and a block ranked by its largest r alone */
 };
 enum { ZG_LM_ROT_PLAIN = 0, ZG_LM_ROT_YARN = 1 /* blend by pair index, amplitude factor */, ZG_LM_ROT_BANDS = 2 /* by wavelength: see rot_* */ };
 typedef struct {
@@ -441,7 +445,7 @@ typedef struct {
     float ff_limit;               /* ZG_LM_ACT_GLU_CLIPPED: the experts' clip */
     int shared_width;             /* > 0: a shared expert of this hidden width (same activation) runs for every token and is added;
                                      with the clipped activation times sigmoid(shared.sg . h) (tensors shared.gate / up / down / sg),
-                                     with ZG_LM_ACT_GLU_SILU as it is (tensors shared.gate / up / down) */
+                                     with ZG_LM_ACT_GLU_SILU as it is (tensors shared.gate / up / down) unless shared_gate says so */
     float shared_limit;           /* its clip */
     /* (the fields below are zero for the designs that do not name them) */
     float tau;                    /* gated linear attention: the decay is sigmoid(.)^(1 / tau) */
@@ -461,6 +465,18 @@ typedef struct {
     int head_gate;                /* latent attention: != 0: head h's output is multiplied by sigmoid(W_g h)_h (tensor `mix.g`) */
     int norm_groups;              /* selective state space: equal parts of the norm behind the gate (0: 1) */
     int dense_act;                /* ZG_LM_DENSE_* */
+    int proj_bias;                /* rotary attention: != 0: q, k, v and o have biases (fp32 tensors mix.q.b, k.b, v.b, o.b) */
+    int value_norm;               /* rotary attention: != 0: every value head is divided by its root mean square over vdim (norm_eps, no
+                                     weight) */
+    int value_mix;                /* rotary attention: != 0: v <- (1 - l) v + l v', l the fp32 scalar mix.vmix, v' the (normed, unmixed) values
+                                     of the same token in the first pass that has this field set (which leaves its own as they are and
+                                     needs no mix.vmix); the mixed values are cached */
+    int sigmoid_weights;          /* rotary attention: != 0: no softmax: a visible key weighs sigmoid(score + mix.pb[h]), nothing is normalised
+                                     over the keys */
+    int sink;                     /* latent attention: != 0: exp(mix.sink[h]) is part of the softmax's denominator */
+    int identity;                 /* ZG_LM_ROUTE_SOFTMAX_GROUPS: pass-through outputs behind the `experts` units: the router has experts + identity
+                                     outputs, and a chosen pass-through output contributes weight * h (no tensors) */
+    int shared_gate;              /* != 0 with ZG_LM_ACT_GLU_SILU: the shared expert times sigmoid(shared.sg . h) */
 } zg_lm_layer;
 enum {
     ZG_LM_F32 = 1 << 0,     /* true 32-bit products everywhere */
@@ -477,8 +493,9 @@ enum {
                                   mixer reads norm1(x) as it is (no token shift, no input convolution), and a sublayer's normed output
                                   enters the residual sum times residual_mult */
     ZG_LM_EMBED_NORM = 1 << 7, /* the embedding output passes the stack's norm with the tensors `embed.norm` (ZG_LM_TANH_NORMS only) */
-    ZG_LM_NO_SHIFT = 1 << 8    /* sequential sublayers with RMS norms whose mixer reads norm1(x) as it is: no token shift, no input
+    ZG_LM_NO_SHIFT = 1 << 8,   /* sequential sublayers with RMS norms whose mixer reads norm1(x) as it is: no token shift, no input
                                   convolution */
+    ZG_LM_LAYER_SCALE = 1 << 9 /* ZG_LM_SIDE_BY_SIDE: x += ls1 * mixer(norm1(x)) + ls2 * ff(norm2(x)), element by element (tensors `ls1`, `ls2`) */
 };
 typedef struct {
     size_t vocab, width, n_layers;
@@ -509,9 +526,10 @@ int zg_lm_destroy(zg_lm* g);
  * right.ri right.ri.b right.lam right.o right.out; delta rule: q q.conv k k.conv v v.conv b A_log dt_bias a1 a2 g1 g2 norm o;
  * window + linear pair: left.q|k|v with .b and .conv each, left.q.norm left.k.norm left.g left.o left.o.b right.q right.k right.v
  * right.g right.norm right.o right.decay; gated linear attention: q k v g o norm a1 a2 a2.b; attention: q k o;
- * rotary attention: q k v o; selective state space: in conv conv.b dt_bias A_log D norm o; latent attention with q_rank 0: q for
- * dq dq.norm uq, with head_gate also g, with kv_from no dkv and dkv.norm)
- * and `l<i>.mlp.*` (dense: up down, and act with a polynomial activation; experts: e<j>.gate e<j>.up e<j>.down router, and correction or router.b; shared.gate shared.up
+ * rotary attention: q k v o, with proj_bias q.b k.b v.b o.b, with sigmoid_weights pb, with value_mix vmix; selective state space: in conv conv.b dt_bias A_log D norm o; latent attention with q_rank 0: q for
+ * dq dq.norm uq, with head_gate also g, with sink also sink, with kv_from no dkv and dkv.norm)
+ * (ZG_LM_LAYER_SCALE: `l<i>.ls1|ls2`)
+ * and `l<i>.mlp.*` (dense: up down, gate with a gated one, and act with a polynomial activation; experts: e<j>.gate e<j>.up e<j>.down router, and correction or router.b; shared.gate shared.up
  * shared.down shared.sg).  data: fp32 on the host, `len` elements, matrices
  * [out][in] row-major; matrices are stored bf16 (round to nearest even).  ZG_ERR_ARG for a name the configuration does not have. */
 int zg_lm_load_tensor(zg_lm* g, const char* name, const float* data, size_t len);

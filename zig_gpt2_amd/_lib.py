@@ -54,7 +54,8 @@ class LmLayer(C.Structure):
                 ("shared_limit", C.c_float), ("tau", C.c_float), ("softcap", C.c_float), ("qtemp_coef", C.c_float), ("qtemp_every", C.c_int),
                 ("dist_bias", C.c_int), ("route_groups", C.c_int), ("route_keep", C.c_int), ("route_scale", C.c_float), ("weights_of", C.c_int),
                 ("rot_halves", C.c_int), ("chunk", C.c_int), ("kv_from", C.c_int), ("head_gate", C.c_int), ("norm_groups", C.c_int),
-                ("dense_act", C.c_int)]
+                ("dense_act", C.c_int), ("proj_bias", C.c_int), ("value_norm", C.c_int), ("value_mix", C.c_int), ("sigmoid_weights", C.c_int),
+                ("sink", C.c_int), ("identity", C.c_int), ("shared_gate", C.c_int)]
 
 
 class LmConfig(C.Structure):
@@ -75,13 +76,13 @@ class LmEntry(C.Structure):
 LM_MIX_HGRN2, LM_MIX_LATENT_ATTENTION, LM_MIX_PARALLEL, LM_MIX_CHANNEL_DELTA, LM_MIX_WINDOW_LINEAR = 1, 2, 3, 4, 5
 LM_MIX_GLA, LM_MIX_ATTENTION, LM_MIX_ROTARY_ATTENTION, LM_MIX_SSD = 6, 7, 8, 9
 LM_FF_NONE, LM_FF_DENSE, LM_FF_MOE = 0, 1, 2
-LM_DENSE_RELU2, LM_DENSE_POLYNORM = 0, 1
+LM_DENSE_RELU2, LM_DENSE_POLYNORM, LM_DENSE_GLU_GELU = 0, 1, 2
 LM_ACT_GLU_SILU, LM_ACT_GELU, LM_ACT_GLU_CLIPPED = 0, 1, 2
 LM_ROUTE_SOFTMAX_ALL, LM_ROUTE_TOP_LOGITS, LM_ROUTE_SIGMOID_INPUT = 0, 1, 2
-LM_ROUTE_SIGMOID_GROUPS = 3
+LM_ROUTE_SIGMOID_GROUPS, LM_ROUTE_SOFTMAX_GROUPS = 3, 4
 LM_ROT_PLAIN, LM_ROT_YARN, LM_ROT_BANDS = 0, 1, 2
 LM_F32, LM_NO_GRAPH, LM_TIED_HEAD, LM_LOOP_READD, LM_SIDE_BY_SIDE, LM_SINUSOID_POSITIONS = 1, 2, 4, 8, 16, 32
-LM_TANH_NORMS, LM_EMBED_NORM, LM_NO_SHIFT = 64, 128, 256
+LM_TANH_NORMS, LM_EMBED_NORM, LM_NO_SHIFT, LM_LAYER_SCALE = 64, 128, 256, 512
 
 # the layered-model tier (present in both libraries)
 LM_SIGNATURES = {

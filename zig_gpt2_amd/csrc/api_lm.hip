@@ -32,6 +32,8 @@
 // A selective state space keeps the tail of its convolution and its [heads][state][vdim] state in the block of sequence state; chunked
 // attention caches rotated keys and plain values like the windowed one (a chunk is a window whose front edge moves by whole chunks).
 // A latent attention layer may read the latents another layer has cached: it then owns no cache, and its pass points at that one's.
+// Rotary attention whose passes mix the first such pass's values into their own passes those along in a scratch row per token (every
+// token runs through all passes in one portion): only the mixed values are cached.
 //
 // Latent attention runs in its absorbed form in prompts and in decoding alike: score_j = (W_uk^T q_nope) . c_j + q_rot . k_rot_j,
 // out = W_uv (sum_j p_j c_j) — only the latent c_j and the rotated key part are cached, and a portion of a prompt needs nothing
@@ -96,6 +98,11 @@ struct LayerW {
     float *a2b = nullptr, *slopes = nullptr;
     // selective state space: the skip factors and the weight of the norm in parts;  polynomial activation: its four numbers
     float *skip = nullptr, *part_norm = nullptr, *poly = nullptr;
+    // side-by-side sublayers: factors per channel of the two results;  rotary attention: head offsets of the sigmoid weights, the factor of
+    // the value mix;  dense feed-forward: rows of its first product (gate | up with a gated activation)
+    float *ls1 = nullptr, *ls2 = nullptr, *gate_bias = nullptr, *vmix = nullptr;
+    int n_up = 0;
+    int ld_sgu = 0;  // row stride of the shared expert's first product
     int ld_cat = 0;  // row stride of the fused projection's output (a multiple of four: 16-byte loads behind it)
 };
 
@@ -104,6 +111,7 @@ struct Pass {
     size_t hgrn_off = 0;     // floats into a slot's recurrent-state block
     float* cache = nullptr;  // latent cache (or key / value cache) of this pass
     bool readd = false;      // the embedding output is added to x in front of this pass
+    bool mix_first = false;  // the first pass that mixes values: its own are kept for the later ones
     // floats into a slot's block of sequence state: tails of the two input convolutions, tail of the mixer's own convolution,
     // the mixer's recurrent state
     size_t canon1_off = 0, canon2_off = 0, conv_off = 0, rec_off = 0;
@@ -204,6 +212,7 @@ struct zg_lm {
     float embed_scale = 1.0f;
     bool side = false;          // ZG_LM_SIDE_BY_SIDE
     bool no_shift = false;      // ZG_LM_NO_SHIFT
+    bool layer_scale = false;   // ZG_LM_LAYER_SCALE
     bool tanh_norms = false;    // ZG_LM_TANH_NORMS: every norm pointer is a block [w | b | alpha]
     float res_mult = 1.0f;      // ... and a sublayer's normed output enters the residual sum times this
     float* embed_norm = nullptr;  // ZG_LM_EMBED_NORM
@@ -218,6 +227,7 @@ struct zg_lm {
     int* amax_idx = nullptr;
     float *attn_ws = nullptr, *scan_ws = nullptr, *win_ws = nullptr;
     size_t win_ws_floats = 0;
+    float* v_first = nullptr;  // [rows][kv_heads vdim]: values of the first pass that mixes them
     float *x0 = nullptr, *hc = nullptr, *y2 = nullptr, *ta = nullptr, *tb = nullptr, *tc = nullptr, *td = nullptr;
     size_t scan_ws_floats = 0;
     size_t attn_ws_floats = 0;
@@ -316,7 +326,7 @@ void layout(zg_lm* g, Bump& b) {
     if (tn) norm3("final.norm", g->final_norm);
     else vec("final.norm", g->final_norm, W, g->side ? INIT_PLAIN : INIT_OFFSET);
     if (g->cfg.flags & ZG_LM_SINUSOID_POSITIONS) g->pos_freq = b.take<float>((W + 1) / 2);
-    size_t max_t = 1, max_win = 0, max_win_few = 0;
+    size_t max_t = 1, max_win = 0, max_win_few = 0, max_vf = 0;
     size_t max_proj = 1, max_qr = 1, max_q = 1, max_qa = 1, max_ctx = 1, max_o = 1, max_ff = 1, max_assign = 1, max_gu = 1, max_hb = 1, max_e = 1, max_att_part = 0, max_scan = 0;
     for (size_t i = 0; i < g->layers.size(); ++i) {
         LayerW& L = g->layers[i];
@@ -333,6 +343,10 @@ void layout(zg_lm* g, Bump& b) {
             if (g->no_shift) {
             } else if (taps == 0) vec(p + "shift", L.shift, W, INIT_UNIT);
             else vec(p + "canon1", L.canon1, W * taps, INIT_OFFSET);
+        }
+        if (g->layer_scale) {
+            vec(p + "ls1", L.ls1, W, INIT_PLAIN);
+            if (d.ff != ZG_LM_FF_NONE) vec(p + "ls2", L.ls2, W, INIT_PLAIN);
         }
         const size_t H = d.heads, D = d.dim, Vd = d.vdim;
         if (d.mixer == ZG_LM_MIX_PARALLEL) {
@@ -483,11 +497,30 @@ void layout(zg_lm* g, Bump& b) {
             L.o = b.take<bf16_t>(W * H * Vd);
             mat(p + "mix.o", L.o, 0, W, H * Vd);
             L.rot_freq = b.take<float>(std::max<size_t>(1, d.rot_dims / 2));
+            if (d.proj_bias) {
+                L.qkv_bias = b.take<float>(NP);
+                vec_at(p + "mix.q.b", L.qkv_bias, 0, HD, INIT_OFFSET);
+                vec_at(p + "mix.k.b", L.qkv_bias, HD, GD, INIT_OFFSET);
+                vec_at(p + "mix.v.b", L.qkv_bias, HD + GD, GV, INIT_OFFSET);
+                vec(p + "mix.o.b", L.obias, W, INIT_OFFSET);
+            }
+            if (d.sigmoid_weights) vec(p + "mix.pb", L.gate_bias, H, INIT_OFFSET);
+            if (d.value_mix) {
+                vec(p + "mix.vmix", L.vmix, 1, INIT_UNIT);
+                int others = 0;  // passes that read it
+                for (const Pass& ps : g->passes) others += ps.layer == (int)i && !ps.mix_first ? 1 : 0;
+                T[p + "mix.vmix"].loaded = others == 0;  // (never missed)
+                max_vf = std::max(max_vf, GV);
+            }
             max_proj = std::max(max_proj, (size_t)L.ld_cat);
             max_o = std::max(max_o, H * Vd);
             const int cap = rotary_key_capacity(g, d);
-            max_win = std::max(max_win, std::min(window_split_workspace((int)MS, (int)H, (int)Vd, cap, nullptr), (size_t)1 << 29));
-            max_win_few = std::max(max_win_few, window_split_workspace(kGemvMaxRows, (int)H, (int)Vd, cap, nullptr));
+            if (d.sigmoid_weights) {
+                max_win_few = std::max(max_win_few, gate_split_workspace((int)H, (int)Vd, cap));
+            } else {
+                max_win = std::max(max_win, std::min(window_split_workspace((int)MS, (int)H, (int)Vd, cap, nullptr), (size_t)1 << 29));
+                max_win_few = std::max(max_win_few, window_split_workspace(kGemvMaxRows, (int)H, (int)Vd, cap, nullptr));
+            }
         } else if (d.mixer == ZG_LM_MIX_SSD) {
             const size_t G = d.kv_heads, HV = H * Vd, CC = HV + 2 * G * D, NP = HV + CC + H;
             L.n_cat = (int)NP;
@@ -532,6 +565,7 @@ void layout(zg_lm* g, Bump& b) {
                 vec(p + "mix.dkv.norm", L.dkv_norm, KR, INIT_PLAIN);
             }
             if (NG) mat(p + "mix.g", L.dqkv, NQ + NL, NG, W);
+            if (d.sink) vec(p + "mix.sink", L.sink, H, INIT_OFFSET);
             if (QR > 0) {
                 vec(p + "mix.dq.norm", L.dq_norm, QR, INIT_PLAIN);
                 L.uq = b.take<bf16_t>(H * (D + R) * QR);
@@ -562,12 +596,16 @@ void layout(zg_lm* g, Bump& b) {
         }
         const size_t F = d.ff_width;
         if (d.ff == ZG_LM_FF_DENSE) {
-            L.up = b.take<bf16_t>(F * W);
-            mat(p + "mlp.up", L.up, 0, F, W);
+            const bool gated = d.dense_act == ZG_LM_DENSE_GLU_GELU;
+            L.n_up = (int)(gated ? 2 * F : F);
+            L.up = b.take<bf16_t>((size_t)L.n_up * W);
+            if (gated) mat(p + "mlp.gate", L.up, 0, F, W);
+            mat(p + "mlp.up", L.up, L.n_up - F, F, W);
             L.down = b.take<bf16_t>(W * F);
             mat(p + "mlp.down", L.down, 0, W, F);
             if (d.dense_act == ZG_LM_DENSE_POLYNORM) vec(p + "mlp.act", L.poly, 4, INIT_PLAIN);
-            max_ff = std::max(max_ff, F);
+            max_ff = std::max(max_ff, (size_t)L.n_up);
+            if (gated) max_hb = std::max(max_hb, F);
         } else if (d.ff == ZG_LM_FF_MOE) {
             const size_t E = d.experts, UF = d.ff_act == ZG_LM_ACT_GELU ? F : 2 * F;  // rows of an expert's first matrix
             L.gu = b.take<bf16_t>(E * UF * W);
@@ -578,19 +616,22 @@ void layout(zg_lm* g, Bump& b) {
                 mat(q + "up", L.gu, e * UF + (UF - F), F, W);
                 mat(q + "down", L.edown, e * W, W, F);
             }
-            L.router = b.take<bf16_t>(E * W);
-            mat(p + "mlp.router", L.router, 0, E, W);
+            const size_t ER = E + d.identity;  // the router's outputs
+            L.router = b.take<bf16_t>(ER * W);
+            mat(p + "mlp.router", L.router, 0, ER, W);
             if (d.router != ZG_LM_ROUTE_SIGMOID_INPUT)
-                vec(p + (d.router == ZG_LM_ROUTE_TOP_LOGITS ? "mlp.router.b" : "mlp.correction"), L.correction, E, INIT_OFFSET);
-            if (d.shared_width > 0) {  // the shared expert: gate | up rows and, behind them, the row of its gate logit (clipped form)
+                vec(p + (d.router == ZG_LM_ROUTE_TOP_LOGITS ? "mlp.router.b" : "mlp.correction"), L.correction, ER, INIT_OFFSET);
+            if (d.shared_width > 0) {  // the shared expert: gate | up rows and, behind them, the row of its gate logit (where it has one)
                 const size_t S = d.shared_width;
+                const bool sg = d.ff_act == ZG_LM_ACT_GLU_CLIPPED || d.shared_gate;
+                L.ld_sgu = (int)(d.ff_act == ZG_LM_ACT_GLU_CLIPPED ? 2 * S + 1 : (2 * S + (sg ? 1 : 0) + 3) & ~(size_t)3);
                 L.sgu = b.take<bf16_t>((2 * S + 1) * W);
                 mat(p + "mlp.shared.gate", L.sgu, 0, S, W);
                 mat(p + "mlp.shared.up", L.sgu, S, S, W);
-                if (d.ff_act == ZG_LM_ACT_GLU_CLIPPED) mat(p + "mlp.shared.sg", L.sgu, 2 * S, 1, W);
+                if (sg) mat(p + "mlp.shared.sg", L.sgu, 2 * S, 1, W);
                 L.sdown = b.take<bf16_t>(W * S);
                 mat(p + "mlp.shared.down", L.sdown, 0, W, S);
-                max_t = std::max(max_t, std::max(2 * S + 1, W));
+                max_t = std::max(max_t, std::max((size_t)L.ld_sgu, W));
             }
             max_assign = std::max(max_assign, (size_t)d.top);
             max_gu = std::max(max_gu, (size_t)d.top * UF);
@@ -697,6 +738,7 @@ void layout(zg_lm* g, Bump& b) {
     if (max_win > ((size_t)1 << 29)) max_win = 0;
     g->win_ws_floats = max_win;
     g->win_ws = b.take<float>(std::max<size_t>(1, max_win));
+    g->v_first = b.take<float>(std::max<size_t>(1, MS * max_vf));
     g->last_h = b.take<float>((size_t)g->n_passes * NS * W);
     g->hn = b.take<float>((size_t)g->logit_rows * W);
     g->logits = b.take<float>((size_t)g->logit_rows * V);
@@ -808,16 +850,16 @@ int check_layer(const zg_lm_layer& d, size_t i, unsigned flags) {
                    "layer %zu: rotary scaling constants must be positive", i);
     }
     ZG_REQUIRE(d.ff == ZG_LM_FF_NONE || d.ff == ZG_LM_FF_DENSE || d.ff == ZG_LM_FF_MOE, ZG_ERR_ARG, "layer %zu: unknown feed-forward %d", i, d.ff);
-    ZG_REQUIRE(d.dense_act == ZG_LM_DENSE_RELU2 || d.dense_act == ZG_LM_DENSE_POLYNORM, ZG_ERR_ARG, "layer %zu: dense activation %d", i, d.dense_act);
+    ZG_REQUIRE(d.dense_act >= ZG_LM_DENSE_RELU2 && d.dense_act <= ZG_LM_DENSE_GLU_GELU, ZG_ERR_ARG, "layer %zu: dense activation %d", i, d.dense_act);
     ZG_REQUIRE(d.kv_from == 0 || (d.mixer == ZG_LM_MIX_LATENT_ATTENTION && d.q_rank == 0), ZG_ERR_UNSUPPORTED,
                "layer %zu: another layer's latents are read by latent attention with directly projected queries", i);
     ZG_REQUIRE(d.head_gate == 0 || (d.mixer == ZG_LM_MIX_LATENT_ATTENTION && d.q_rank == 0), ZG_ERR_UNSUPPORTED,
                "layer %zu: the gate per head is built for latent attention with directly projected queries", i);
     ZG_REQUIRE(d.ff == ZG_LM_FF_NONE || d.ff_width >= 1, ZG_ERR_ARG, "layer %zu: feed-forward width %d", i, d.ff_width);
-    ZG_REQUIRE(d.ff != ZG_LM_FF_MOE || (d.experts >= 1 && d.experts <= 256 && d.top >= 1 && d.top <= d.experts), ZG_ERR_UNSUPPORTED,
+    ZG_REQUIRE(d.ff != ZG_LM_FF_MOE || (d.experts >= 1 && d.experts <= 256 && d.top >= 1 && d.top <= d.experts + std::max(0, d.identity)), ZG_ERR_UNSUPPORTED,
                "layer %zu: %d experts, %d chosen (at most 256 experts)", i, d.experts, d.top);
     ZG_REQUIRE(d.ff_act >= ZG_LM_ACT_GLU_SILU && d.ff_act <= ZG_LM_ACT_GLU_CLIPPED && d.router >= ZG_LM_ROUTE_SOFTMAX_ALL &&
-                   d.router <= ZG_LM_ROUTE_SIGMOID_GROUPS,
+                   d.router <= ZG_LM_ROUTE_SOFTMAX_GROUPS,
                ZG_ERR_ARG, "layer %zu: expert activation %d, router rule %d", i, d.ff_act, d.router);
     if (d.ff == ZG_LM_FF_MOE && !(flags & ZG_LM_SIDE_BY_SIDE))
         ZG_REQUIRE(d.ff_act != ZG_LM_ACT_GLU_CLIPPED && d.router != ZG_LM_ROUTE_SIGMOID_INPUT && (d.shared_width == 0 || (flags & ZG_LM_TANH_NORMS)),
@@ -825,16 +867,25 @@ int check_layer(const zg_lm_layer& d, size_t i, unsigned flags) {
                    "layer %zu: the clipped activation and the input-weighted router are built for side-by-side sublayers, a shared expert for those or "
                    "for the norms without statistics",
                    i);
-    if (d.ff == ZG_LM_FF_MOE && d.router == ZG_LM_ROUTE_SIGMOID_GROUPS) {
-        const int ng = std::max(1, d.route_groups), nk = d.route_keep >= 1 ? d.route_keep : ng;
-        ZG_REQUIRE(d.experts % ng == 0 && nk <= ng && d.top <= nk * (d.experts / ng) && d.route_scale >= 0.0f, ZG_ERR_ARG,
-                   "layer %zu: %d experts in %d groups, %d groups kept, %d chosen, weight factor %g", i, d.experts, ng, nk, d.top, d.route_scale);
+    ZG_REQUIRE(d.identity == 0 || (d.identity > 0 && d.ff == ZG_LM_FF_MOE && d.router == ZG_LM_ROUTE_SOFTMAX_GROUPS && (flags & ZG_LM_SIDE_BY_SIDE) &&
+                                   d.experts + d.identity <= 256),
+               ZG_ERR_UNSUPPORTED, "layer %zu: %d pass-through outputs beside %d experts (softmax router with groups, side-by-side sublayers, at most 256 together)",
+               i, d.identity, d.experts);
+    if (d.ff == ZG_LM_FF_MOE && (d.router == ZG_LM_ROUTE_SIGMOID_GROUPS || d.router == ZG_LM_ROUTE_SOFTMAX_GROUPS)) {
+        const int ng = std::max(1, d.route_groups), nk = d.route_keep >= 1 ? d.route_keep : ng, ne = d.experts + d.identity;
+        ZG_REQUIRE(ne % ng == 0 && nk <= ng && d.top <= nk * (ne / ng) && d.route_scale >= 0.0f, ZG_ERR_ARG,
+                   "layer %zu: %d experts in %d groups, %d groups kept, %d chosen, weight factor %g", i, ne, ng, nk, d.top, d.route_scale);
     }
+    ZG_REQUIRE(d.mixer == ZG_LM_MIX_ROTARY_ATTENTION || (!d.proj_bias && !d.value_norm && !d.value_mix && !d.sigmoid_weights), ZG_ERR_UNSUPPORTED,
+               "layer %zu: projection biases, normed or mixed values and sigmoid weights are built for rotary attention", i);
+    ZG_REQUIRE(!d.sink || d.mixer == ZG_LM_MIX_LATENT_ATTENTION, ZG_ERR_UNSUPPORTED, "layer %zu: the sink of this field is built for latent attention", i);
+    ZG_REQUIRE(!d.shared_gate || ((flags & ZG_LM_SIDE_BY_SIDE) && d.ff_act == ZG_LM_ACT_GLU_SILU), ZG_ERR_UNSUPPORTED,
+               "layer %zu: the gate of a shared expert with silu units is built for side-by-side sublayers", i);
     if (d.ff == ZG_LM_FF_MOE && d.ff_act == ZG_LM_ACT_GLU_CLIPPED)
         ZG_REQUIRE(d.ff_limit > 0.0f && (d.shared_width == 0 || d.shared_limit > 0.0f), ZG_ERR_ARG, "layer %zu: clip %g (shared expert: %g)", i, d.ff_limit,
                    d.shared_limit);
     ZG_REQUIRE(d.shared_width >= 0 && (d.shared_width == 0 || d.ff_act == ZG_LM_ACT_GLU_CLIPPED ||
-                                       (d.ff_act == ZG_LM_ACT_GLU_SILU && (flags & ZG_LM_TANH_NORMS))),
+                                       (d.ff_act == ZG_LM_ACT_GLU_SILU && (flags & (ZG_LM_TANH_NORMS | ZG_LM_SIDE_BY_SIDE)))),
                ZG_ERR_UNSUPPORTED, "layer %zu: a shared expert needs a gated activation", i);
     return ZG_OK;
 }
@@ -881,10 +932,21 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
     // the dense feed-forward of a layer: in -> out
     auto dense_ff = [&](const LayerW& L, const float* in, float* out) -> int {
         const int F = L.d.ff_width;
-        const bool poly = L.d.dense_act == ZG_LM_DENSE_POLYNORM;
+        const bool poly = L.d.dense_act == ZG_LM_DENSE_POLYNORM, gated = L.d.dense_act == ZG_LM_DENSE_GLU_GELU;
         Linear up, dn;
-        up.A = in; up.lda = W; up.B = L.up; up.ldb = W; up.C = g->u; up.ldc = F; up.M = M; up.N = F; up.K = W; up.act = poly ? ACT_NONE : ACT_RELU2;
+        up.A = in; up.lda = W; up.B = L.up; up.ldb = W; up.C = g->u; up.ldc = L.n_up; up.M = M; up.N = L.n_up; up.K = W;
+        up.act = poly || gated ? ACT_NONE : ACT_RELU2;
         ZG_TRY(launch_linear(up, f32, s));
+        if (gated) {  // rows gate | up
+            dn.B = L.down; dn.ldb = F; dn.C = out; dn.ldc = W; dn.M = M; dn.N = W; dn.K = F;
+            if (M <= 2) {  // the activation where the second product reads its rows (more rows: every workgroup would redo it)
+                dn.A = g->u; dn.lda = L.n_up; dn.a_glu = F; dn.glu_kind = GLU_GELU;
+            } else {
+                ZG_TRY(launch_glu(g->u, g->hb, M, F, s, GLU_GELU));
+                dn.A = g->hb; dn.lda = F;
+            }
+            return launch_linear(dn, f32, s);
+        }
         if (poly && M <= kPolyMaxRows) {  // decode steps: the activation where the second product reads its rows
             dn.a_poly = L.poly;
             dn.poly_eps = eps;
@@ -945,20 +1007,40 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             mask.window = d.window;
             mask.chunk = d.chunk;
             lin.A = hin; lin.lda = W; lin.B = L.wcat; lin.ldb = W; lin.C = g->proj; lin.ldc = LD; lin.M = M; lin.N = L.n_cat; lin.K = W;
+            lin.bias = L.qkv_bias;
             ZG_TRY(launch_linear(lin, f32, s));
-            ZG_TRY(launch_window_prep(g->proj, LD, M, H, G, D, Vd, rot, nullptr, d_pos, d_slot, g->page_table, g->max_pages, g->P, ps.cache, s));
+            ValuePrep vals;
+            vals.norm = d.value_norm != 0;
+            vals.eps = eps;
+            if (d.value_mix && ps.mix_first) vals.first_out = g->v_first;
+            else if (d.value_mix) vals.mix_first = g->v_first, vals.lam = L.vmix;
             const int cap = rotary_key_capacity(g, d);
             // (a bounded layer's decode steps take its bound at any length)
             const int key_cap = (d.chunk > 0 || d.window > 0) && (single || capturing) ? cap : std::min(cap, whole_context_keys(single || capturing));
-            bool split = false;
-            ZG_TRY(launch_window_attention_split(g->proj, LD, g->o, HV, M, H, G, D, Vd, d.scale, mask, nullptr, nullptr, nullptr, d_pos, d_slot,
-                                                 g->page_table, g->max_pages, g->P, ps.cache, key_cap, g->win_ws, g->win_ws_floats, d_estart, d_elen,
-                                                 n_ent, s, &split));
-            if (!split)
+            bool done = false;
+            auto gated = [&](const Rotary* fused) {
+                return launch_gate_attention(g->proj, LD, g->o, HV, M, H, G, D, Vd, d.scale, L.gate_bias, mask, f32, fused, vals, d_pos, d_slot,
+                                             g->page_table, g->max_pages, g->P, ps.cache, key_cap, g->win_ws, g->win_ws_floats, d_estart, d_elen, n_ent,
+                                             s, &done);
+            };
+            if (d.sigmoid_weights && single) ZG_TRY(gated(&rot));  // decode steps: the rows' preparation inside the attention's launch
+            if (!done) {
+                ZG_TRY(launch_window_prep(g->proj, LD, M, H, G, D, Vd, rot, nullptr, d_pos, d_slot, g->page_table, g->max_pages, g->P, ps.cache, s, vals));
+                if (d.sigmoid_weights) ZG_TRY(gated(nullptr));
+                else
+                    ZG_TRY(launch_window_attention_split(g->proj, LD, g->o, HV, M, H, G, D, Vd, d.scale, mask, nullptr, nullptr, nullptr, d_pos, d_slot,
+                                                         g->page_table, g->max_pages, g->P, ps.cache, key_cap, g->win_ws, g->win_ws_floats, d_estart,
+                                                         d_elen, n_ent, s, &done));
+            }
+            if (!done) {
+                ScoreShape shape;
+                shape.gate = L.gate_bias;
                 ZG_TRY(launch_window_attention(g->proj, LD, g->o, HV, M, H, G, D, Vd, d.scale, mask, nullptr, nullptr, nullptr, d_pos, d_slot,
-                                               g->page_table, g->max_pages, g->P, ps.cache, s));
+                                               g->page_table, g->max_pages, g->P, ps.cache, s, shape));
+            }
             lin = Linear();
             lin.A = g->o; lin.lda = HV; lin.B = L.o; lin.ldb = HV; lin.C = g->y; lin.ldc = W; lin.M = M; lin.N = W; lin.K = HV;
+            lin.bias = L.obias;
             ZG_TRY(launch_linear(lin, f32, s));
         } else if (d.mixer == ZG_LM_MIX_SSD) {
             const int G = d.kv_heads, HV = H * Vd, CC = HV + 2 * G * D, LD = L.ld_cat;
@@ -1156,10 +1238,10 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             bool tiled = false;
             if (!f32 && !few)
                 ZG_TRY(launch_latent_attention_tiles(g->qa, g->ctx, M, H, KR, R, d.scale, d_estart, d_elen, d_eslot, n_ent, d_pos, g->page_table,
-                                                     g->max_pages, g->P, ps.cache, s, &tiled, gate, LD));
+                                                     g->max_pages, g->P, ps.cache, s, &tiled, gate, LD, L.sink));
             if (!tiled)
                 ZG_TRY(launch_latent_attention(g->qa, g->ctx, M, H, KR, R, d.scale, d_pos, d_slot, g->page_table, g->max_pages, g->P, ps.cache,
-                                               g->attn_ws, g->attn_ws_floats, s, gate, LD));
+                                               g->attn_ws, g->attn_ws_floats, s, gate, LD, L.sink));
             lin = Linear();  // values of the weighted latent, head by head
             lin.A = g->ctx; lin.lda = H * KR; lin.a_zoff = KR; lin.B = L.uv; lin.ldb = KR; lin.b_zoff = (long long)Vd * KR;
             lin.C = g->o; lin.ldc = HV; lin.c_zoff = Vd; lin.M = M; lin.N = Vd; lin.K = KR; lin.nz = H;
@@ -1262,7 +1344,8 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
                 const int E = d.experts, top = d.top, NA = M * top;
                 const int UF = d.ff_act == ZG_LM_ACT_GELU ? F : 2 * F;
                 const bool on_input = d.router == ZG_LM_ROUTE_SIGMOID_INPUT;  // the router's score multiplies the expert's input
-                ZG_TRY(launch_route(fin, M, W, L.router, L.correction, E, top, g->pick, g->wt, d.router, s, d.route_groups, d.route_keep,
+                const int* passes_through = d.identity > 0 ? g->pick : nullptr;  // choices that stand for the input itself
+                ZG_TRY(launch_route(fin, M, W, L.router, L.correction, E + d.identity, top, g->pick, g->wt, d.router, s, d.route_groups, d.route_keep,
                                     d.route_scale != 0.0f ? d.route_scale : 1.0f));
                 Linear up, dn;
                 up.A = fin; up.lda = W; up.a_div = top; up.B = L.gu; up.ldb = W; up.b_zoff = (long long)UF * W; up.C = g->gu_buf; up.ldc = UF;
@@ -1271,16 +1354,29 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
                 dn.A = g->hb; dn.lda = F; dn.B = L.edown; dn.ldb = F; dn.b_zoff = (long long)W * F; dn.C = g->ye; dn.ldc = W; dn.N = W; dn.K = F;
                 if (few) {  // one batch per assignment, its expert's matrices looked up on the device
                     up.M = dn.M = 1; up.nz = dn.nz = NA; up.z_group = dn.z_group = g->pick;
+                    up.z_limit = dn.z_limit = E;
                     up.c_zoff = UF; dn.c_zoff = W;
                 } else {  // assignments sorted by expert, grouped products
                     ZG_TRY(launch_group(g->pick, NA, E, g->grp_off, g->sorted, g->inv, s));
                     up.M = dn.M = NA; up.a_rows = g->sorted; up.grp_off = dn.grp_off = g->grp_off; up.n_groups = dn.n_groups = E;
                 }
-                ZG_TRY(launch_linear(up, f32, s));
+                const bool silu = d.ff_act == ZG_LM_ACT_GLU_SILU;
+                const int S = d.shared_width, sg_col = d.shared_gate ? 2 * S : -1, SL = L.ld_sgu;
+                const bool paired = few && silu && S > 0;
+                Linear sup, sdn;  // steps of few rows: the expert every token uses rides in the chosen experts' launches, a batch per row
+                if (paired) {
+                    sup.A = fin; sup.lda = W; sup.a_zoff = W; sup.B = L.sgu; sup.ldb = W; sup.C = g->tb; sup.ldc = SL; sup.c_zoff = SL;
+                    sup.M = 1; sup.nz = M; sup.N = 2 * S + (sg_col >= 0 ? 1 : 0); sup.K = W;
+                    ZG_TRY(launch_linear_pair(up, sup, f32, s));
+                } else {
+                    ZG_TRY(launch_linear(up, f32, s));
+                }
                 // (the product is linear: the score that multiplies an expert's input is applied to the product, in front of the clip)
                 if (d.ff_act == ZG_LM_ACT_GELU) {
                     dn.A = g->gu_buf; dn.lda = F;
-                } else if (d.ff_act == ZG_LM_ACT_GLU_SILU) {
+                } else if (silu && few) {  // the activation is applied where the second product reads its rows
+                    dn.A = g->gu_buf; dn.lda = 2 * F; dn.a_glu = F;
+                } else if (silu) {
                     ZG_TRY(launch_glu(g->gu_buf, g->hb, NA, F, s));
                 } else if (few) {  // the activation is applied where the second product reads its rows
                     dn.A = g->gu_buf; dn.lda = 2 * F; dn.a_glu = F; dn.glu_kind = GLU_CLIPPED; dn.glu_limit = d.ff_limit;
@@ -1288,10 +1384,25 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
                 } else {
                     ZG_TRY(launch_glu_clipped(g->gu_buf, UF, g->hb, NA, F, d.ff_limit, on_input ? g->wt : nullptr, g->sorted, -1, s));
                 }
-                ZG_TRY(launch_linear(dn, f32, s));
                 const float* ys = nullptr;
-                if (d.shared_width > 0) {  // the shared expert; its gate logit is the last column of its first product
-                    const int S = d.shared_width;
+                if (paired) {
+                    sdn.A = g->tb; sdn.lda = SL; sdn.a_zoff = SL; sdn.a_glu = S; sdn.glu_gate_col = sg_col; sdn.B = L.sdown; sdn.ldb = S; sdn.C = g->td;
+                    sdn.ldc = W; sdn.c_zoff = W; sdn.M = 1; sdn.nz = M; sdn.N = W; sdn.K = S;
+                    ZG_TRY(launch_linear_pair(dn, sdn, f32, s));
+                    ys = g->td;
+                } else {
+                    ZG_TRY(launch_linear(dn, f32, s));
+                }
+                if (S > 0 && silu && !paired) {
+                    lin = Linear();
+                    lin.A = fin; lin.lda = W; lin.B = L.sgu; lin.ldb = W; lin.C = g->tb; lin.ldc = SL; lin.M = M; lin.N = 2 * S + (sg_col >= 0 ? 1 : 0); lin.K = W;
+                    ZG_TRY(launch_linear(lin, f32, s));
+                    ZG_TRY(launch_glu(g->tb, g->tc, M, S, s, GLU_SILU, SL, sg_col));
+                    lin = Linear();
+                    lin.A = g->tc; lin.lda = S; lin.B = L.sdown; lin.ldb = S; lin.C = g->td; lin.ldc = W; lin.M = M; lin.N = W; lin.K = S;
+                    ZG_TRY(launch_linear(lin, f32, s));
+                    ys = g->td;
+                } else if (S > 0 && !silu) {  // the shared expert; its gate logit is the last column of its first product
                     lin = Linear();
                     lin.A = fin; lin.lda = W; lin.B = L.sgu; lin.ldb = W; lin.C = g->tb; lin.ldc = 2 * S + 1; lin.M = M; lin.N = 2 * S + 1; lin.K = W;
                     ZG_TRY(launch_linear(lin, f32, s));
@@ -1311,8 +1422,11 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
                     pend.exp_w = on_input ? nullptr : g->wt;
                     pend.top = top;
                     pend.b = ys;
+                    pend.pick = passes_through;
+                    pend.n_exp = E;
+                    pend.ident = fin;
                 } else {
-                    ZG_TRY(launch_expert_sum(g->y2, g->ye, g->inv, on_input ? nullptr : g->wt, top, ys, M, W, s));
+                    ZG_TRY(launch_expert_sum(g->y2, g->ye, g->inv, on_input ? nullptr : g->wt, top, ys, M, W, s, passes_through, E, fin));
                     pend.b = g->y2;
                 }
             }
@@ -1320,6 +1434,10 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             if (d.ff == ZG_LM_FF_DENSE) pend.b = g->y2;
             pend.bias = d.mixer == ZG_LM_MIX_WINDOW_LINEAR ? L.obias : nullptr;
             pend.w = d.left_scale;
+            if (g->layer_scale) {
+                pend.sa = L.ls1;
+                pend.sb = L.ls2;
+            }
             if (p + 1 == g->n_passes || (g->trace && !capturing)) {  // nobody behind to add them (or the stream is to be shown): add now
                 ZG_TRY(launch_add_two(g->x, pend, M, W, s));
                 pend = OpenSums();
@@ -1624,6 +1742,7 @@ int zg_lm_create(zg_lm** out, const zg_lm_config* config, int device) {
     g->side = (config->flags & ZG_LM_SIDE_BY_SIDE) != 0;
     g->tanh_norms = (config->flags & ZG_LM_TANH_NORMS) != 0;
     g->no_shift = (config->flags & ZG_LM_NO_SHIFT) != 0;
+    g->layer_scale = (config->flags & ZG_LM_LAYER_SCALE) != 0;
     g->res_mult = config->residual_mult != 0.0f ? config->residual_mult : 1.0f;
     g->embed_scale = config->embed_scale != 0.0f ? config->embed_scale : 1.0f;
     int status = ZG_OK;
@@ -1651,7 +1770,7 @@ int zg_lm_create(zg_lm** out, const zg_lm_config* config, int device) {
         if (status == ZG_OK && j != i) {
             const zg_lm_layer &a = g->layers[i].d, &o = g->layers[j].d;
             if (a.mixer != o.mixer || a.heads != o.heads || a.dim != o.dim || a.vdim != o.vdim || a.kv_heads != o.kv_heads || a.ff != o.ff ||
-                a.ff_width != o.ff_width || a.experts != o.experts || a.top != o.top || a.shared_width != o.shared_width) {
+                a.ff_width != o.ff_width || a.experts != o.experts || a.top != o.top || a.shared_width != o.shared_width || a.identity != o.identity) {
                 set_error("lm_create: layer %zu names the weights of layer %zu, whose sizes differ", i, j);
                 status = ZG_ERR_ARG;
             }
@@ -1665,6 +1784,23 @@ int zg_lm_create(zg_lm** out, const zg_lm_config* config, int device) {
             d.weights_of > 0 || g->layers[j].d.kv_rank != d.kv_rank || g->layers[j].d.rot_dim != d.rot_dim) {
             set_error("lm_create: layer %zu reads the latents of layer %zu, which must lie in front of it with latents of its own of the same sizes", i, j);
             status = ZG_ERR_ARG;
+        }
+    }
+    if (status == ZG_OK && g->layer_scale && !g->side) {
+        set_error("lm_create: factors per channel on a sublayer's result are built for side-by-side sublayers");
+        status = ZG_ERR_UNSUPPORTED;
+    }
+    {  // passes that mix values pass rows of one shape along
+        int first = -1;
+        for (size_t i = 0; i < config->n_layers && status == ZG_OK; ++i) {
+            const zg_lm_layer& d = g->layers[owner[i]].d;
+            if (!d.value_mix) continue;
+            if (first < 0) first = (int)i;
+            const zg_lm_layer& f = g->layers[owner[first]].d;
+            if (d.kv_heads != f.kv_heads || d.vdim != f.vdim) {
+                set_error("lm_create: layer %zu mixes values of %d x %d channels into its own of %d x %d", i, f.kv_heads, f.vdim, d.kv_heads, d.vdim);
+                status = ZG_ERR_ARG;
+            }
         }
     }
     if (status == ZG_OK && g->no_shift && (g->side || g->tanh_norms || g->canon != 0)) {
@@ -1713,6 +1849,11 @@ int zg_lm_create(zg_lm** out, const zg_lm_config* config, int device) {
         }
     for (int i = (k > 1 ? b : 0); i < n; ++i) add(i);
     g->n_passes = (int)g->passes.size();
+    for (Pass& ps : g->passes)
+        if (g->layers[ps.layer].d.value_mix) {
+            ps.mix_first = true;
+            break;
+        }
     // how far back any attention pass looks: pages behind that are given back while a sequence is still open
     bool attends = false, bounded = true;
     for (const Pass& ps : g->passes) {

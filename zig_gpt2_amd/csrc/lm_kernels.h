@@ -17,7 +17,11 @@ namespace lm {
 // ------------------------------------------------------------------------------------------------ linear maps
 enum { ACT_NONE = 0, ACT_RELU2 = 1, ACT_GELU_ERF = 2, ACT_SCALE_SOFTCAP = 3 /* v <- v act_a, then act_b tanh(v / act_b) when act_b > 0 */ };
 // Gated activations of rows [gate (F) | up (F)] (GLU_CLIPPED: also a row factor and the clip `limit`)
-enum { GLU_SILU = 0 /* silu(gate) up */, GLU_CLIPPED = 1 /* g sigmoid(1.702 g) (u + 1), g = min(s gate, limit), u = clamp(s up, -limit, limit) */ };
+enum {
+    GLU_SILU = 0 /* silu(gate) up */,
+    GLU_CLIPPED = 1 /* g sigmoid(1.702 g) (u + 1), g = min(s gate, limit), u = clamp(s up, -limit, limit) */,
+    GLU_GELU = 2 /* gelu(gate) up, the tanh form */
+};
 
 // C[m][n] = act( sum_k A[arow(m)][k] * B[n][k] )      for m < M, n < N
 //   arow(m) = a_rows ? a_rows[m] / a_div : m          (row gather: a token's row feeds each of its expert assignments)
@@ -37,6 +41,7 @@ struct Linear {
     int M = 0, N = 0, K = 0;
     int act = ACT_NONE;
     float act_a = 1.0f, act_b = 0.0f;  // constants of ACT_SCALE_SOFTCAP
+    const float* bias = nullptr;       // [N]: added to the product in front of `act` (the same for every batch)
     int a_glu = 0;  // > 0 (row-vector kernel only): A rows are [gate (a_glu) | up (a_glu)] and enter through their gated activation, K = a_glu
     int glu_kind = GLU_SILU;
     float glu_limit = 0.0f;            // GLU_CLIPPED
@@ -47,6 +52,7 @@ struct Linear {
     int nz = 1;
     long long a_zoff = 0, b_zoff = 0, c_zoff = 0;
     const int* z_group = nullptr;
+    int z_limit = 0x7fffffff;  // batches whose z_group is not below it are skipped, their rows of C left alone (row-vector kernels)
     const int* grp_off = nullptr;
     int n_groups = 0;
 };
@@ -89,14 +95,20 @@ int launch_sum_norm_shift(float* x, const float* y, const float* yexp, const flo
 // out[j] = x[rows[j]] / rms * (1 + w)            (the model's last norm on the rows whose logits are asked for; plain: * w)
 int launch_norm_gather(const float* x, const int* rows, const float* w, float eps, float* out, int n_rows, int W, bool plain, hipStream_t s);
 // Side-by-side sublayers: both read the same x through norms with plain weights, so one pass serves both:
-//   [x[m] += add.a[m] + add.b[m] + add.w * add.bias + sum_k (add.exp_w ? add.exp_w[m top + k] : 1) add.exp[m top + k]
-//    (what the layer before left open; any part may be null)]
+//   [x[m] += sa * (add.a[m] + add.w * add.bias) + sb * (add.b[m] + sum_k (add.exp_w ? add.exp_w[m top + k] : 1) add.exp[m top + k])
+//    (what the layer before left open; any part may be null; sa, sb: factors per channel, null: 1)]
 //   ha[m] = x[m] / rms(x[m]) * wa;   hb[m] = x[m] / rms(x[m]) * wb   (hb / wb may be null)
 struct OpenSums {
     const float *a = nullptr, *b = nullptr, *bias = nullptr;
     float w = 0.0f;
     const float *exp = nullptr, *exp_w = nullptr;  // rows of the chosen experts in assignment order, `top` per token
     int top = 0;
+    const float *sa = nullptr, *sb = nullptr;
+    // pass-through choices: an assignment whose pick is not below n_exp has no row in exp and stands for ident[m] (needs exp_w).  ident
+    // may be the launch's own hb: an element is read by the thread that later writes it.
+    const int* pick = nullptr;
+    int n_exp = 0;
+    const float* ident = nullptr;
     __host__ __device__ bool any() const { return a || b || bias || exp; }
 };
 int launch_norm_two(float* x, const OpenSums& add, const float* wa, const float* wb, float eps, float* ha, float* hb, int M, int W, hipStream_t s);
@@ -222,16 +234,18 @@ int launch_q_rotary(const float* q, int ldq, float* qa, int ldqa, int M, int H, 
 // ws: fp32 workspace for the partials of split key ranges (steps of at most kGemvMaxRows rows: M * H * kAttnSplits * (KR + 2)
 // floats; without it whole key rows per workgroup).
 // gate != null: head h's result is multiplied by sigmoid(gate[m ldg + h]).
+// sink != null: exp(sink[h]) is added to head h's denominator, once.
 constexpr int kAttnSplits = 16;
 int launch_latent_attention(const float* qa, float* ctx, int M, int H, int KR, int R, float scale, const int* row_pos, const int* row_slot,
                             const int* page_table, int max_pages, int page_tokens, const float* cache, float* ws, size_t ws_floats, hipStream_t s,
-                            const float* gate = nullptr, int ldg = 0);
+                            const float* gate = nullptr, int ldg = 0, const float* sink = nullptr);
 
 // The same for prompt portions on the matrix cores (bf16 operands, fp32 scores / softmax / accumulation): 32 queries of one entry
 // and four heads per workgroup.  *taken = false when the latent is larger than the kernel's tiles hold (nothing launched).
 int launch_latent_attention_tiles(const float* qa, float* ctx, int M, int H, int KR, int R, float scale, const int* ent_start, const int* ent_len,
                                   const int* ent_slot, int n_entries, const int* row_pos, const int* page_table, int max_pages, int page_tokens,
-                                  const float* cache, hipStream_t s, bool* taken, const float* gate = nullptr, int ldg = 0);
+                                  const float* cache, hipStream_t s, bool* taken, const float* gate = nullptr, int ldg = 0,
+                                  const float* sink = nullptr);
 
 // ------------------------------------------------------------------------------------------------ input convolution of decode rows, residual sum
 // Steps of one row per entry: [x += x0] or [x += norm(y) * (1 + wb), y = yl or the mean of the two normed branches yl, yr with
@@ -247,9 +261,19 @@ int launch_add_rows(float* x, const float* y, int M, int W, hipStream_t s);
 // proj rows [q (H D) | k (G D) | v (G V)]: q rotated in place; the rotated key and the value rotated over all V channels (pair i by
 // pos * vfreq[i]) written to the token's cache row [G D | G V]; the page of (slot, pos) is page_table[slot][(pos / P) % max_pages]:
 // a ring, so that a sequence whose old pages have been given back can grow beyond max_pages * P positions.
-// vfreq == null: the values are cached as they are.
+// vfreq == null: the values are cached as they are, or as `vals` says (vfreq == null only).
+// What becomes of a value head on its way into the cache: [v <- v / rms(v) over its V channels], [written to first_out as well],
+// [v <- (1 - *lam) v + *lam mix_first[m]].
+struct ValuePrep {
+    bool norm = false;
+    float eps = 0.0f;
+    float* first_out = nullptr;        // [M][G V]
+    const float* mix_first = nullptr;  // [M][G V]
+    const float* lam = nullptr;
+};
 int launch_window_prep(float* proj, int ld, int M, int H, int G, int D, int V, Rotary rot, const float* vfreq, const int* row_pos,
-                       const int* row_slot, const int* page_table, int max_pages, int page_tokens, float* cache, hipStream_t s);
+                       const int* row_slot, const int* page_table, int max_pages, int page_tokens, float* cache, hipStream_t s,
+                       const ValuePrep& vals = ValuePrep());
 // out[m][h] = turn_back_pos( sum_j w_h(j) value_(h / (H/G))(j) ),  w_h = sum_g talk[h][g] p_g,
 // p_g(j) = exp(s_g(j)) / (exp(sink_g) + sum_j' exp(s_g(j'))),  s_g(j) = scale q_g . k(j),  over the keys pos - window < j <= pos
 // (window 0: all j <= pos; chunk > 0: the keys of pos's own chunk [n chunk, (n + 1) chunk) up to pos).  sink / talk may be null (no
@@ -257,10 +281,12 @@ int launch_window_prep(float* proj, int ld, int M, int H, int G, int D, int V, R
 // keep_first > 0: beyond the window the first keep_first positions of the sequence stay visible (a row's keys are then numbered
 // kept tokens first, then the window).  vfreq == null: values are cached unrotated and nothing is turned back.
 // shape: what becomes of a scaled score before the softmax — capped (cap > 0: cap tanh(s / cap)), then less slope[h] per position
-// of distance between the query and the key (slope != null).
+// of distance between the query and the key (slope != null).  gate != null: no softmax: the weight of a key is sigmoid(score + gate[h])
+// (no sink, no statistics).
 struct ScoreShape {
     float cap = 0.0f;
     const float* slope = nullptr;  // [H]
+    const float* gate = nullptr;   // [H]
 };
 // which keys at or before a query it sees: a sliding window (with the sequence's first keep tokens behind it), its chunk, or all
 struct KeyMask {
@@ -300,6 +326,20 @@ int launch_window_attention_split(const float* q, int ldq, float* out, int ldo, 
                                   const float* out_gate = nullptr, int ld_gate = 0, float out_factor = 1.0f, ScoreShape shape = ScoreShape());
 // (out_gate != null: a taken step multiplies the result by sigmoid(out_gate[m][.]) * out_factor where the shares are added)
 
+// ------------------------------------------------------------------------------------------------ attention with sigmoid weights
+// out[m][h] = sum_j sigmoid(scale q_h . k(j) + bias[h]) value(j) over the keys the mask shows (windows and chunks; no kept tokens), q rows
+// and cache rows as above, nothing normalised over the keys: two kernels instead of the three passes of the softmax forms.
+// rot != null (steps of one row per entry): q rows are the raw projection [q | k | v]; the launch also does what launch_window_prep
+// would (rotary q, the token's cache row with `vals` applied to its values) — q itself is left as it was.
+// f32: prompt portions multiply in true fp32 instead of with bf16 operands.
+// ws: gate_split_workspace floats (partial sums of long key ranges in steps of few rows; too small: one workgroup walks the range).
+// *taken = false (nothing launched) for heads of more than 256 channels: launch_window_attention with ScoreShape::gate.
+size_t gate_split_workspace(int H, int V, int key_capacity);
+int launch_gate_attention(const float* q, int ldq, float* out, int ldo, int M, int H, int G, int D, int V, float scale, const float* bias, KeyMask mask,
+                          bool f32, const Rotary* rot, const ValuePrep& vals, const int* row_pos, const int* row_slot, const int* page_table,
+                          int max_pages, int page_tokens, float* cache, int key_capacity, float* ws, size_t ws_floats, const int* ent_start,
+                          const int* ent_len, int n_entries, hipStream_t s, bool* taken);
+
 // ------------------------------------------------------------------------------------------------ real-gated linear recurrent unit
 // Per entry and channel c: r = sigmoid(gr + br), i = sigmoid(gi + bi), a = exp(-8 r softplus(lam)), S = a S + sqrt(1 - a^2) i u,
 // out = S * gelu_tanh(y + by); S = state[slot][c], read at the start of the entry and written back at its end.
@@ -333,6 +373,8 @@ int launch_norm_gate(float* v, int ld, int rows_per_m, int width, int M, const f
 // contiguous blocks of equal size, a block ranks by r of its best plus r of its second-best expert, experts outside the `keep`
 // top-ranked blocks get r = -inf; the `top` highest r win (lowest index wins a tie); weights s / (sum of the winners' s + 1e-20)
 // * out_scale.
+// rule ZG_LM_ROUTE_SOFTMAX_GROUPS: the same with s = softmax(z) and a block ranked by its best r alone.
+// E counts the router's outputs, pass-through ones included.
 // pre != null (norms without statistics, widths up to kRouteFuseWidth): the routing workgroup of a row first does what
 // launch_tanh_sum_norm would — x[m] += mult * nb(sum of y's parts), h[m] = nn(x[m]) with h == g — and routes on the result.
 struct RoutePre {
@@ -347,9 +389,11 @@ constexpr int kRouteFuseWidth = 8192;
 int launch_route(const float* g, int M, int W, const bf16_t* router, const float* correction, int E, int top, int* pick, float* weight,
                  int rule, hipStream_t s, int groups = 1, int keep = 1, float out_scale = 1.0f, const RoutePre* pre = nullptr);
 // Sort the M * top assignments by expert: grp_off[E + 1], sorted[p] = assignment at sorted position p, inv[a] = position of a.
+// Picks that are not below E (pass-through outputs) lie behind grp_off[E].
 int launch_group(const int* pick, int n_assign, int E, int* grp_off, int* sorted, int* inv, hipStream_t s);
-// h[p][j] = silu(gu[p][j]) * gu[p][F + j]
-int launch_glu(const float* gu, float* h, int rows, int F, hipStream_t s);
+// h[p][j] = act(gu[p][j]) * gu[p][F + j] * t, act by kind (GLU_SILU, GLU_GELU), gu rows ld floats apart (0: 2 F)
+//   t = gate_col >= 0 ? sigmoid(gu[p][gate_col]) : 1        (a gate logit that the same product left in the row)
+int launch_glu(const float* gu, float* h, int rows, int F, hipStream_t s, int kind = GLU_SILU, int ld = 0, int gate_col = -1);
 // h[p][j] = act(s gu[p][j], s gu[p][F + j]) * t,  act(g, u) = g' sigmoid(1.702 g') (u' + 1), g' = min(g, limit), u' = clamp(u, -limit, limit)
 //   s = row_scale ? row_scale[row_of ? row_of[p] : p] : 1   (the router's score of the assignment that sits at sorted place p)
 //   t = gate_col >= 0 ? sigmoid(gu[p][gate_col]) : 1        (a gate logit that the same product left in the row)
@@ -357,7 +401,9 @@ int launch_glu(const float* gu, float* h, int rows, int F, hipStream_t s);
 int launch_glu_clipped(const float* gu, int ld, float* h, int rows, int F, float limit, const float* row_scale, const int* row_of, int gate_col,
                        hipStream_t s);
 // y[m] = sum_k (weight ? weight[m top + k] : 1) * yexp[inv ? inv[m top + k] : m top + k] (+ ys[m]), in choice order
-int launch_expert_sum(float* y, const float* yexp, const int* inv, const float* weight, int top, const float* ys, int M, int W, hipStream_t s);
+// pick != null: assignments whose pick is not below n_exp take ident[m] instead of a row of yexp
+int launch_expert_sum(float* y, const float* yexp, const int* inv, const float* weight, int top, const float* ys, int M, int W, hipStream_t s,
+                      const int* pick = nullptr, int n_exp = 0, const float* ident = nullptr);
 // y = sum_k weight[m][k] * yexp[inv ? inv[m top + k] : m top + k];   x[m] += y / rms(y) * (1 + w)
 int launch_moe_combine(float* x, const float* yexp, const int* inv, const float* weight, int top, const float* w, float eps, int M, int W,
                        hipStream_t s);

@@ -37,6 +37,8 @@ struct LinArgs {
     int M, N, K;
     int a_div, act, n_groups, a_glu;
     float act_a, act_b;
+    const float* bias;
+    int z_limit;
     int glu_kind;
     float glu_limit;
     const float* glu_scale;
@@ -46,8 +48,10 @@ struct LinArgs {
     int a_vec, b_vec;  // 16-byte loads allowed (alignment of base, leading dimension and batch offsets)
 };
 
-__device__ __forceinline__ float apply_act(float v, const LinArgs& p) {
+// output n on its way out: the bias, then the activation
+__device__ __forceinline__ float finish(float v, int n, const LinArgs& p) {
     const int act = p.act;
+    if (p.bias) v += p.bias[n];
     if (act == ACT_SCALE_SOFTCAP) {
         v *= p.act_a;
         if (p.act_b > 0.0f) v = p.act_b * tanhf(v / p.act_b);
@@ -67,6 +71,7 @@ __device__ __forceinline__ float glu_on_load(float g, float u, const LinArgs& p,
         u = fminf(fmaxf(u * sc, -p.glu_limit), p.glu_limit);
         return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
     }
+    if (p.glu_kind == GLU_GELU) return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
     return g / (1.0f + expf(-g)) * u;
 }
 
@@ -135,6 +140,7 @@ __device__ __forceinline__ void gemv_body(const LinArgs& p, const int z) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n0 = blockIdx.x * 8 + wave * 2;
     if (n0 >= p.N) return;
+    if (p.z_group && p.z_group[z] >= p.z_limit) return;
     const bf16_t* B = p.B + (long long)(p.z_group ? p.z_group[z] : z) * p.b_zoff;
     const float* A = p.A + (long long)z * p.a_zoff;
     float* C = p.C + (long long)z * p.c_zoff;
@@ -218,8 +224,8 @@ __device__ __forceinline__ void gemv_body(const LinArgs& p, const int z) {
         }
         const float s0 = POLY ? acc0[m] : wave_allsum(acc0[m]), s1 = POLY ? acc1[m] : wave_allsum(acc1[m]);
         if (lane == 0 && m < p.M) {
-            C[(long long)m * p.ldc + n0] = apply_act(s0, p);
-            if (two) C[(long long)m * p.ldc + n0 + 1] = apply_act(s1, p);
+            C[(long long)m * p.ldc + n0] = finish(s0, n0, p);
+            if (two) C[(long long)m * p.ldc + n0 + 1] = finish(s1, n0 + 1, p);
         }
     }
 }
@@ -245,6 +251,7 @@ __global__ __launch_bounds__(256) void lm_gemv_ks_kernel(const LinArgs p) {
     __shared__ float s_part[4][MR][POLY ? 11 : 2];
     const int z = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n0 = blockIdx.x * 2;
+    if (p.z_group && p.z_group[z] >= p.z_limit) return;
     const bf16_t* B = p.B + (long long)(p.z_group ? p.z_group[z] : z) * p.b_zoff;
     const float* A = p.A + (long long)z * p.a_zoff;
     float* C = p.C + (long long)z * p.c_zoff;
@@ -329,7 +336,7 @@ __global__ __launch_bounds__(256) void lm_gemv_ks_kernel(const LinArgs p) {
             const int m = threadIdx.x >> 1, c = threadIdx.x & 1;
             auto sum4 = [&](int i) { return (s_part[0][m][i] + s_part[1][m][i]) + (s_part[2][m][i] + s_part[3][m][i]); };
             const float d[4] = {sum4(3 + 4 * c), sum4(4 + 4 * c), sum4(5 + 4 * c), sum4(6 + 4 * c)};
-            if (m < p.M && n0 + c < p.N) C[(long long)m * p.ldc + n0 + c] = apply_act(poly_value(p, sum4(0), sum4(1), sum4(2), d), p);
+            if (m < p.M && n0 + c < p.N) C[(long long)m * p.ldc + n0 + c] = finish(poly_value(p, sum4(0), sum4(1), sum4(2), d), n0 + c, p);
         }
         return;
     }
@@ -345,7 +352,7 @@ __global__ __launch_bounds__(256) void lm_gemv_ks_kernel(const LinArgs p) {
     if (threadIdx.x < MR * 2) {
         const int m = threadIdx.x >> 1, c = threadIdx.x & 1;
         if (m < p.M && n0 + c < p.N)
-            C[(long long)m * p.ldc + n0 + c] = apply_act((s_part[0][m][c] + s_part[1][m][c]) + (s_part[2][m][c] + s_part[3][m][c]), p);
+            C[(long long)m * p.ldc + n0 + c] = finish((s_part[0][m][c] + s_part[1][m][c]) + (s_part[2][m][c] + s_part[3][m][c]), n0 + c, p);
     }
 }
 
@@ -525,7 +532,7 @@ __global__ __launch_bounds__(256) void lm_gemm_kernel(const LinArgs p) {
 #pragma unroll
             for (int e = 0; e < 16; ++e) {
                 const int m = m0 + (wy * WT + i) * 32 + 8 * (e >> 2) + 4 * (lane >> 5) + (e & 3);
-                if (m < m_end) C[(long long)m * p.ldc + n] = apply_act(acc[i][j][e], p);
+                if (m < m_end) C[(long long)m * p.ldc + n] = finish(acc[i][j][e], n, p);
             }
         }
 }
@@ -559,7 +566,7 @@ LinArgs make_args(const Linear& L) {
     p.a_zoff = L.a_zoff; p.b_zoff = L.b_zoff; p.c_zoff = L.c_zoff;
     p.lda = L.lda; p.ldb = L.ldb; p.ldc = L.ldc; p.M = L.M; p.N = L.N; p.K = L.K;
     p.a_div = L.a_div; p.act = L.act; p.n_groups = L.grp_off ? L.n_groups : 0; p.a_glu = L.a_glu;
-    p.act_a = L.act_a; p.act_b = L.act_b; p.glu_kind = L.glu_kind; p.glu_limit = L.glu_limit; p.glu_scale = L.glu_scale;
+    p.act_a = L.act_a; p.act_b = L.act_b; p.bias = L.bias; p.z_limit = L.z_limit; p.glu_kind = L.glu_kind; p.glu_limit = L.glu_limit; p.glu_scale = L.glu_scale;
     p.glu_gate_col = L.glu_gate_col;
     p.a_poly = L.a_poly;
     p.poly_eps = L.poly_eps;
@@ -601,6 +608,7 @@ int launch_linear(const Linear& L, bool f32, hipStream_t s) {
     }
     ZG_REQUIRE(L.a_glu == 0, ZG_ERR_ARG, "linear: the gated activation on load is for steps of few rows");
     ZG_REQUIRE(!(L.z_group && L.grp_off), ZG_ERR_ARG, "linear: a matrix per batch and row groups exclude each other");
+    ZG_REQUIRE(L.z_limit == 0x7fffffff, ZG_ERR_ARG, "linear: skipped batches are for steps of few rows");
     // 64 x 64 tiles.  The 128 x 128 form of the same kernel measured slower at every size tried (a prompt pass of 8 x 1023
     // tokens at width 1600: 143 against 127 ms; width 768: 14.6 against 12.9 ms) and is kept behind ZGPT2_LM_GEMM_TILE=128 only
     // (tests run ragged shapes through it).

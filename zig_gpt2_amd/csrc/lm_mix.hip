@@ -261,18 +261,27 @@ __global__ __launch_bounds__(256) void norm_gather_kernel(const float* x, const 
 // Side-by-side sublayers: the residual sum the layer before left open, then the two norms of the same row from one statistic.
 // Rows of up to 256 * kRowRegs floats stay in registers between the statistic and the results.
 __device__ __forceinline__ float open_sums_at(const OpenSums& add, size_t m, int i, int W, float v) {
-    if (add.a) v += add.a[m * W + i];
+    if (add.sa) {  // a factor per channel on either sublayer's result
+        float a = add.a ? add.a[m * W + i] : 0.0f;
+        if (add.bias) a = fmaf(add.w, add.bias[i], a);
+        v = fmaf(add.sa[i], a, v);
+    } else if (add.a) {
+        v += add.a[m * W + i];
+    }
+    const float sb = add.sb ? add.sb[i] : 1.0f;
     if (add.exp) {  // in choice order: the sum does not depend on the batch
         float e = 0.0f;
         for (int k = 0; k < add.top; ++k) {
-            const float y = add.exp[(m * add.top + k) * W + i];
-            e = add.exp_w ? fmaf(add.exp_w[m * add.top + k], y, e) : e + y;
+            const size_t as = m * add.top + k;
+            const float y = add.pick && add.pick[as] >= add.n_exp ? add.ident[m * W + i] : add.exp[as * W + i];
+            e = add.exp_w ? fmaf(add.exp_w[as], y, e) : e + y;
         }
-        v += add.b ? e + add.b[m * W + i] : e;
+        if (add.b) e += add.b[m * W + i];
+        v = fmaf(sb, e, v);
     } else if (add.b) {
-        v += add.b[m * W + i];
+        v = fmaf(sb, add.b[m * W + i], v);
     }
-    if (add.bias) v = fmaf(add.w, add.bias[i], v);
+    if (add.bias && !add.sa) v = fmaf(add.w, add.bias[i], v);
     return v;
 }
 
@@ -824,12 +833,22 @@ __global__ __launch_bounds__(256) void latent_direct_prep_kernel(const float* pr
 // With n_split > 1 (decode steps: few rows, long key ranges) grid.z workgroups share a row's keys in ranges of at least 64
 // and leave (maximum, sum, weighted latent) partials in ws for latent_merge_kernel.
 // gate (may be null): head h's result is multiplied by sigmoid(gate[m ldg + h]) where it is written.
+// 1 / (L + exp(sink - mx)) times what brings weights of reference point mx to that denominator's (L: sum of exp(score - mx); mx -inf:
+// no keys).  sink null: 1 / L.
+__device__ __forceinline__ float sink_norm_f(float mx, float L, const float* sink, int h) {
+    if (!sink) return 1.0f / L;
+    const float s = sink[h];
+    if (s <= mx) return 1.0f / (L + expf(s - mx));
+    const float e = expf(mx - s);
+    return e / (L * e + 1.0f);
+}
 __device__ __forceinline__ float head_gate_f(const float* gate, int ldg, size_t m, int h) { return gate ? sigmoid_f(gate[m * ldg + h]) : 1.0f; }
 
 template <int ND>
 __global__ __launch_bounds__(256) void latent_attention_kernel(const float* qa, float* ctx, int H, int KR, int R, float scale, const int* row_pos,
                                                                const int* row_slot, const int* page_table, int max_pages, int page_tokens,
-                                                               const float* cache, float* ws, int n_split, const float* gate, int ldg) {
+                                                               const float* cache, float* ws, int n_split, const float* gate, int ldg,
+                                                               const float* sink) {
     __shared__ float s_m[4], s_l[4];
     __shared__ float s_acc[4][ND * 64];
     const int m = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -915,12 +934,12 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const float* qa, 
         return;
     }
     float* out = ctx + ((size_t)m * H + h) * KR;
-    const float gf = head_gate_f(gate, ldg, m, h);
+    const float gf = head_gate_f(gate, ldg, m, h) * (sink ? sink_norm_f(M4, L, sink, h) : 1.0f);
     for (int d = threadIdx.x; d < KR; d += blockDim.x) {
         float a = 0.0f;
 #pragma unroll
         for (int w = 0; w < 4; ++w) a = fmaf(wgt[w], s_acc[w][d], a);
-        out[d] = a / L * gf;
+        out[d] = sink ? a * gf : a / L * gf;
     }
 }
 
@@ -938,7 +957,7 @@ template <int NKS, int NT>  // 16 NKS >= KR + R (score dimensions), 32 NT >= KR 
 __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(const float* qa, float* ctx, int H, int KR, int R, float scale,
                                                                     const int* ent_start, const int* ent_len, const int* ent_slot, int n_entries,
                                                                     const int* row_pos, const int* page_table, int max_pages, int page_tokens,
-                                                                    const float* cache, const float* gate, int ldg) {
+                                                                    const float* cache, const float* gate, int ldg, const float* sink) {
     constexpr int DTp = NKS * 16, KS_LD = DTp + 8, VT_LD = 40;
     __shared__ __attribute__((aligned(16))) bf16_t Ks[32 * KS_LD];
     __shared__ __attribute__((aligned(16))) bf16_t Vt[NT * 32 * VT_LD];
@@ -1092,22 +1111,22 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(const float*
     const float L = lsum + __shfl_xor(lsum, 32, 64);
     if (!q_ok) return;
     float* out = ctx + ((size_t)(m_first + r) * H + h) * KR;
-    const float gf = head_gate_f(gate, ldg, (size_t)(m_first + r), h);
+    const float gf = head_gate_f(gate, ldg, (size_t)(m_first + r), h) * (sink ? sink_norm_f(mx, L, sink, h) : 1.0f);
 #pragma unroll
     for (int t = 0; t < NT; ++t)
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
             const int d = t * 32 + 8 * (i >> 2) + 4 * hf + (i & 3);
-            if (d < KR) out[d] = o[t][i] / L * gf;
+            if (d < KR) out[d] = sink ? o[t][i] * gf : o[t][i] / L * gf;
         }
 }
 
 // ctx[m][h] from the partials of latent_attention_kernel, in a fixed order (the result does not depend on timing); only the
 // ranges that held keys are read
 __global__ __launch_bounds__(256) void latent_merge_kernel(const float* ws, float* ctx, int H, int KR, int n_split, const int* row_pos, const float* gate,
-                                                           int ldg) {
+                                                           int ldg, const float* sink) {
     __shared__ float s_w[64];
-    __shared__ float s_L;
+    __shared__ float s_L, s_M;
     const int m = blockIdx.x, h = blockIdx.y, n_keys = row_pos[m] + 1;
     int chunk = (n_keys + n_split - 1) / n_split;
     chunk = max(64, (chunk + 15) & ~15);
@@ -1120,15 +1139,18 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const float* ws, floa
         const float w = pm == -INFINITY ? 0.0f : expf(pm - M);
         s_w[sidx] = w;
         const float L = wave_allsum(sidx < used ? w * part[(size_t)sidx * (KR + 2) + 1] : 0.0f);
-        if (sidx == 0) s_L = L;
+        if (sidx == 0) {
+            s_L = L;
+            s_M = M;
+        }
     }
     __syncthreads();
     float* out = ctx + ((size_t)m * H + h) * KR;
-    const float L = s_L, gf = head_gate_f(gate, ldg, m, h);
+    const float L = s_L, gf = head_gate_f(gate, ldg, m, h) * (sink ? sink_norm_f(s_M, L, sink, h) : 1.0f);
     for (int d = threadIdx.x; d < KR; d += blockDim.x) {
         float a = 0.0f;
         for (int sidx = 0; sidx < used; ++sidx) a = fmaf(s_w[sidx], part[(size_t)sidx * (KR + 2) + 2 + d], a);
-        out[d] = a / L * gf;
+        out[d] = sink ? a * gf : a / L * gf;
     }
 }
 
@@ -1415,14 +1437,14 @@ int launch_q_rotary(const float* q, int ldq, float* qa, int ldqa, int M, int H, 
 
 int launch_latent_attention_tiles(const float* qa, float* ctx, int M, int H, int KR, int R, float scale, const int* ent_start, const int* ent_len,
                                   const int* ent_slot, int n_entries, const int* row_pos, const int* page_table, int max_pages, int page_tokens,
-                                  const float* cache, hipStream_t s, bool* taken, const float* gate, int ldg) {
+                                  const float* cache, hipStream_t s, bool* taken, const float* gate, int ldg, const float* sink) {
     *taken = false;
     if (M <= 0 || n_entries <= 0) return ZG_OK;
     const int DT = KR + R;
     const dim3 grid((M + 31) / 32 + n_entries, (H + 3) / 4);
 #define ZG_ATT_T(NKS_, NT_)                                                                                                                      \
     latent_attention_mfma_kernel<NKS_, NT_><<<grid, 256, 0, s>>>(qa, ctx, H, KR, R, scale, ent_start, ent_len, ent_slot, n_entries, row_pos, page_table, \
-                                                                 max_pages, page_tokens, cache, gate, ldg)
+                                                                 max_pages, page_tokens, cache, gate, ldg, sink)
     if (DT <= 96 && KR <= 64) ZG_ATT_T(6, 2);
     else if (DT <= 160 && KR <= 128) ZG_ATT_T(10, 4);
     else if (DT <= 288 && KR <= 256) ZG_ATT_T(18, 8);
@@ -1436,7 +1458,7 @@ int launch_latent_attention_tiles(const float* qa, float* ctx, int M, int H, int
 
 int launch_latent_attention(const float* qa, float* ctx, int M, int H, int KR, int R, float scale, const int* row_pos, const int* row_slot,
                             const int* page_table, int max_pages, int page_tokens, const float* cache, float* ws, size_t ws_floats,
-                            hipStream_t s, const float* gate, int ldg) {
+                            hipStream_t s, const float* gate, int ldg, const float* sink) {
     if (M <= 0) return ZG_OK;
     const int nd = (KR + R + 63) / 64;
     ZG_REQUIRE(nd <= 16, ZG_ERR_UNSUPPORTED, "latent attention: %d cached dimensions per token (at most 1024)", KR + R);
@@ -1447,7 +1469,7 @@ int launch_latent_attention(const float* qa, float* ctx, int M, int H, int KR, i
     const dim3 grid(M, H, n_split);
 #define ZG_ATT(ND_)                                                                                                                           \
     latent_attention_kernel<ND_><<<grid, 256, 0, s>>>(qa, ctx, H, KR, R, scale, row_pos, row_slot, page_table, max_pages, page_tokens, cache, ws, \
-                                                      n_split, gate, ldg)
+                                                      n_split, gate, ldg, sink)
     if (nd <= 1) ZG_ATT(1);
     else if (nd <= 2) ZG_ATT(2);
     else if (nd <= 3) ZG_ATT(3);
@@ -1459,7 +1481,7 @@ int launch_latent_attention(const float* qa, float* ctx, int M, int H, int KR, i
 #undef ZG_ATT
     ZG_HIP(hipGetLastError());
     if (n_split > 1) {
-        latent_merge_kernel<<<dim3(M, H), 256, 0, s>>>(ws, ctx, H, KR, n_split, row_pos, gate, ldg);
+        latent_merge_kernel<<<dim3(M, H), 256, 0, s>>>(ws, ctx, H, KR, n_split, row_pos, gate, ldg, sink);
         ZG_HIP(hipGetLastError());
     }
     return ZG_OK;

@@ -30,7 +30,8 @@ __device__ __forceinline__ float block_allsum(float v, float* s_red) {
 // logits alone.
 // sigmoid scores with groups: experts ranked by r = sigmoid(z) + correction; a block of adjacent experts ranks by its best r plus
 // its second-best r, only the `keep` top-ranked blocks (lowest index wins a tie) remain eligible; the weights are the winners'
-// sigmoid(z) over their sum, times out_scale.
+// sigmoid(z) over their sum, times out_scale.  softmax scores with groups (rule 4): the same with the softmax over all outputs for
+// the sigmoid and a block ranked by its best r alone.
 // pre.x != null: the workgroup first finishes its own row — x += mult * nb(sum of the sublayer's parts), h = nn(x), both written
 // out, h also kept in the LDS — and routes on that (steps of few rows: the sum and norm in front of the router need no launch
 // of their own).
@@ -97,10 +98,21 @@ __global__ __launch_bounds__(256) void route_kernel(const float* g, int M, int W
         if (lane == 0) s_z[e] = a;
     }
     __syncthreads();
-    if (rule == 3 && groups > 1) {  // every block's rank, by all four waves: its best r plus its second-best r
+    const bool by_group = rule == 3 || rule == 4, softmax_s = rule == 4;
+    float z_top = 0.0f, z_den = 1.0f;  // softmax scores: every wave forms the statistics itself
+    if (softmax_s) {
+        z_top = -INFINITY;
+        for (int e = lane; e < E; e += 64) z_top = fmaxf(z_top, s_z[e]);
+        z_top = wave_allmax(z_top);
+        z_den = 0.0f;
+        for (int e = lane; e < E; e += 64) z_den += expf(s_z[e] - z_top);
+        z_den = wave_allsum(z_den);
+    }
+    auto score = [&](float v) { return softmax_s ? expf(v - z_top) / z_den : 1.0f / (1.0f + expf(-v)); };
+    if (by_group && groups > 1) {  // every block's rank, by all four waves
         __shared__ float s_c[kMaxExperts];
         const int gsz = E / groups;
-        for (int e = threadIdx.x; e < E; e += blockDim.x) s_c[e] = 1.0f / (1.0f + expf(-s_z[e])) + (correction ? correction[e] : 0.0f);
+        for (int e = threadIdx.x; e < E; e += blockDim.x) s_c[e] = score(s_z[e]) + (correction ? correction[e] : 0.0f);
         __syncthreads();
         for (int gi = threadIdx.x; gi < groups; gi += blockDim.x) {
             float a = -INFINITY, b = -INFINITY;
@@ -113,7 +125,7 @@ __global__ __launch_bounds__(256) void route_kernel(const float* g, int M, int W
                     b = c;
                 }
             }
-            s_gs[gi] = gsz > 1 ? a + b : a;
+            s_gs[gi] = gsz > 1 && !softmax_s ? a + b : a;
         }
         __syncthreads();
     }
@@ -163,12 +175,12 @@ __global__ __launch_bounds__(256) void route_kernel(const float* g, int M, int W
             if (lane + 64 * i < top) weight[(size_t)m * top + lane + 64 * i] = ek[i] / sum;
         return;
     }
-    if (rule == 3) {
+    if (by_group) {
         int pk[4] = {0, 0, 0, 0};  // 1 + the place of the expert among the chosen
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int e = lane + 64 * i;
-            sc[i] = e < E ? 1.0f / (1.0f + expf(-z[i])) : 0.0f;
+            sc[i] = e < E ? score(z[i]) : 0.0f;
             ch[i] = e < E ? sc[i] + (correction ? correction[e] : 0.0f) : -INFINITY;
         }
         if (groups > 1) {
@@ -260,10 +272,11 @@ __global__ __launch_bounds__(256) void route_kernel(const float* g, int M, int W
 // one workgroup: histogram, offsets, placement.  The order inside a group is arbitrary: every row of a grouped product is
 // computed independently of its neighbours, so the results do not depend on it.
 __global__ __launch_bounds__(1024) void group_kernel(const int* pick, int n_assign, int E, int* grp_off, int* sorted, int* inv) {
-    __shared__ int s_cnt[kMaxExperts], s_off[kMaxExperts + 1], s_cur[kMaxExperts];
-    for (int e = threadIdx.x; e < E; e += blockDim.x) s_cnt[e] = s_cur[e] = 0;
+    // (group E gathers the picks that are no expert's: behind the last group, no product visits them)
+    __shared__ int s_cnt[kMaxExperts + 1], s_off[kMaxExperts + 1], s_cur[kMaxExperts + 1];
+    for (int e = threadIdx.x; e <= E; e += blockDim.x) s_cnt[e] = s_cur[e] = 0;
     __syncthreads();
-    for (int a = threadIdx.x; a < n_assign; a += blockDim.x) atomicAdd(&s_cnt[pick[a]], 1);
+    for (int a = threadIdx.x; a < n_assign; a += blockDim.x) atomicAdd(&s_cnt[min(pick[a], E)], 1);
     __syncthreads();
     if (threadIdx.x == 0) {
         int o = 0;
@@ -276,20 +289,23 @@ __global__ __launch_bounds__(1024) void group_kernel(const int* pick, int n_assi
     __syncthreads();
     for (int e = threadIdx.x; e <= E; e += blockDim.x) grp_off[e] = s_off[e];
     for (int a = threadIdx.x; a < n_assign; a += blockDim.x) {
-        const int e = pick[a];
+        const int e = min(pick[a], E);
         const int p = s_off[e] + atomicAdd(&s_cur[e], 1);
         sorted[p] = a;
         inv[a] = p;
     }
 }
 
-__global__ __launch_bounds__(256) void glu_kernel(const float* gu, float* h, size_t n, int F) {
+__global__ __launch_bounds__(256) void glu_kernel(const float* gu, int ld, float* h, size_t n, int F, int kind, int gate_col) {
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= n) return;
     const size_t r = idx / F;
     const int j = (int)(idx % F);
-    const float a = gu[r * 2 * F + j], b = gu[r * 2 * F + F + j];
-    h[idx] = a / (1.0f + expf(-a)) * b;
+    const float* row = gu + r * ld;
+    const float a = row[j], b = row[F + j];
+    float v = kind == GLU_GELU ? 0.5f * a * (1.0f + tanhf(0.7978845608028654f * (a + 0.044715f * a * a * a))) * b : a / (1.0f + expf(-a)) * b;
+    if (gate_col >= 0) v *= 1.0f / (1.0f + expf(-row[gate_col]));
+    h[idx] = v;
 }
 
 // the clipped gated activation: the gate capped from above, the linear part clipped on both sides and lifted by one
@@ -313,7 +329,7 @@ __global__ __launch_bounds__(256) void glu_clipped_kernel(const float* gu, int l
 }
 
 __global__ __launch_bounds__(256) void expert_sum_kernel(float* y, const float* yexp, const int* inv, const float* weight, int top, const float* ys,
-                                                         size_t n, int W) {
+                                                         size_t n, int W, const int* pick, int n_exp, const float* ident) {
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= n) return;
     const size_t m = idx / W;
@@ -321,7 +337,7 @@ __global__ __launch_bounds__(256) void expert_sum_kernel(float* y, const float* 
     float a = 0.0f;
     for (int k = 0; k < top; ++k) {  // in choice order: the sum does not depend on the batch
         const size_t as = m * top + k;
-        const float v = yexp[(size_t)(inv ? inv[as] : as) * W + i];
+        const float v = pick && pick[as] >= n_exp ? ident[idx] : yexp[(size_t)(inv ? inv[as] : as) * W + i];
         a = weight ? fmaf(weight[as], v, a) : a + v;
     }
     if (ys) a += ys[idx];
@@ -376,10 +392,11 @@ int launch_group(const int* pick, int n_assign, int E, int* grp_off, int* sorted
     return ZG_OK;
 }
 
-int launch_glu(const float* gu, float* h, int rows, int F, hipStream_t s) {
+int launch_glu(const float* gu, float* h, int rows, int F, hipStream_t s, int kind, int ld, int gate_col) {
     const size_t n = (size_t)rows * F;
     if (n == 0) return ZG_OK;
-    glu_kernel<<<(unsigned)((n + 255) / 256), 256, 0, s>>>(gu, h, n, F);
+    ZG_REQUIRE(kind == GLU_SILU || kind == GLU_GELU, ZG_ERR_ARG, "gated activation: kind %d", kind);
+    glu_kernel<<<(unsigned)((n + 255) / 256), 256, 0, s>>>(gu, ld > 0 ? ld : 2 * F, h, n, F, kind, gate_col);
     ZG_HIP(hipGetLastError());
     return ZG_OK;
 }
@@ -393,10 +410,12 @@ int launch_glu_clipped(const float* gu, int ld, float* h, int rows, int F, float
     return ZG_OK;
 }
 
-int launch_expert_sum(float* y, const float* yexp, const int* inv, const float* weight, int top, const float* ys, int M, int W, hipStream_t s) {
+int launch_expert_sum(float* y, const float* yexp, const int* inv, const float* weight, int top, const float* ys, int M, int W, hipStream_t s,
+                      const int* pick, int n_exp, const float* ident) {
     const size_t n = (size_t)M * W;
     if (n == 0) return ZG_OK;
-    expert_sum_kernel<<<(unsigned)((n + 255) / 256), 256, 0, s>>>(y, yexp, inv, weight, top, ys, n, W);
+    ZG_REQUIRE(!pick || ident, ZG_ERR_ARG, "expert sum: pass-through choices need the rows they stand for");
+    expert_sum_kernel<<<(unsigned)((n + 255) / 256), 256, 0, s>>>(y, yexp, inv, weight, top, ys, n, W, pick, n_exp, ident);
     ZG_HIP(hipGetLastError());
     return ZG_OK;
 }

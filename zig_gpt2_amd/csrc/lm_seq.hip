@@ -243,10 +243,16 @@ __global__ __launch_bounds__(256) void norm_conv_single_kernel(float* x, const f
 // ------------------------------------------------------------------------------------------------ windowed attention
 // proj rows: [q (H D) | k (G D) | v (G V)].  q is rotated in place (pairs (2i, 2i + 1) below rot.dims, or (i, i + dims / 2)); the
 // rotated key and the value rotated over ALL its channels (pair i by pos * vfreq[i]; vfreq null: as it is) go to the token's cache
-// row [G D | G V].
+// row [G D | G V].  vals: what becomes of the value heads otherwise (a wave per head).
+__device__ __forceinline__ float prepare_value(float v, float r, size_t at, const ValuePrep& vals, float lam) {
+    v *= r;
+    if (vals.first_out) vals.first_out[at] = v;
+    return vals.mix_first ? fmaf(lam, vals.mix_first[at], (1.0f - lam) * v) : v;
+}
+
 __global__ __launch_bounds__(256) void window_prep_kernel(float* proj, int ld, int H, int G, int D, int V, Rotary rot, const float* vfreq,
                                                           const int* row_pos, const int* row_slot, const int* page_table, int max_pages,
-                                                          int page_tokens, float* cache) {
+                                                          int page_tokens, float* cache, const ValuePrep vals) {
     const int m = blockIdx.x;
     const int pos = row_pos[m];
     const int page = page_table[(size_t)row_slot[m] * max_pages + (pos / page_tokens) % max_pages];
@@ -280,6 +286,21 @@ __global__ __launch_bounds__(256) void window_prep_kernel(float* proj, int ld, i
         crow[idx] = out;
     }
     const float* v = k + (size_t)G * D;
+    if (vals.norm || vals.first_out || vals.mix_first) {
+        const int lane = threadIdx.x & 63;
+        const float lam = vals.mix_first ? *vals.lam : 0.0f;
+        for (int g = threadIdx.x >> 6; g < G; g += 4) {
+            float r = 1.0f;
+            if (vals.norm) {
+                float ss = 0.0f;
+                for (int i = lane; i < V; i += 64) ss = fmaf(v[g * V + i], v[g * V + i], ss);
+                r = 1.0f / sqrtf(wave_allsum(ss) / (float)V + vals.eps);
+            }
+            for (int i = lane; i < V; i += 64)
+                crow[(size_t)G * D + g * V + i] = prepare_value(v[g * V + i], r, ((size_t)m * G + g) * V + i, vals, lam);
+        }
+        return;
+    }
     for (int idx = threadIdx.x; idx < G * V; idx += blockDim.x) {
         const int i = idx % V;
         if (!vfreq) {
@@ -313,10 +334,12 @@ __device__ __forceinline__ KeySpan key_span(int pos, const KeyMask& mask) {
 }
 __device__ __forceinline__ int key_pos(const KeySpan& k, int n) { return n < k.n_first ? n : k.j_lo + (n - k.n_first); }
 
-// a scaled score on its way to the softmax: capped, then less the head's slope per position of distance (fp32)
+// a scaled score on its way to the softmax: capped, then less the head's slope per position of distance (fp32); with a gate the
+// result is the key's weight itself
 __device__ __forceinline__ float shape_score(float sc, const ScoreShape& sh, int h, int dist) {
     if (sh.cap > 0.0f) sc = sh.cap * tanhf(sc / sh.cap);
     if (sh.slope) sc -= sh.slope[h] * (float)dist;
+    if (sh.gate) sc = sigmoid_f(sc + sh.gate[h]);
     return sc;
 }
 
@@ -376,7 +399,7 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const float* q, i
         __syncthreads();
     };
 
-    for (int t0 = 0; t0 < n_keys; t0 += kWinTile) {  // pass 1: maximum and denominator per head
+    for (int t0 = shape.gate ? n_keys : 0; t0 < n_keys; t0 += kWinTile) {  // pass 1: maximum and denominator per head
         const int nt = min(kWinTile, n_keys - t0);
         tile_scores(t0, nt);
         for (int h = wave; h < H; h += 4) {
@@ -394,7 +417,7 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const float* q, i
         tile_scores(t0, nt);
         for (int idx = tid; idx < H * kWinTile; idx += blockDim.x) {
             const int h = idx / kWinTile, jj = idx % kWinTile;
-            s_s[idx] = jj < nt ? expf(s_s[idx] - s_max[h]) / s_den[h] : 0.0f;
+            s_s[idx] = jj >= nt ? 0.0f : shape.gate ? s_s[idx] : expf(s_s[idx] - s_max[h]) / s_den[h];
         }
         __syncthreads();
         for (int idx = tid; idx < H * kWinTile; idx += blockDim.x) {
@@ -1330,10 +1353,12 @@ int launch_norm_conv_single(float* x, const float* x0, const float* yl, const fl
 }
 
 int launch_window_prep(float* proj, int ld, int M, int H, int G, int D, int V, Rotary rot, const float* vfreq, const int* row_pos,
-                       const int* row_slot, const int* page_table, int max_pages, int page_tokens, float* cache, hipStream_t s) {
+                       const int* row_slot, const int* page_table, int max_pages, int page_tokens, float* cache, hipStream_t s, const ValuePrep& vals) {
     if (M <= 0) return ZG_OK;
+    ZG_REQUIRE(!(vfreq && (vals.norm || vals.first_out || vals.mix_first)) && (!vals.mix_first || vals.lam), ZG_ERR_ARG,
+               "windowed attention: rotated values are neither normed nor mixed");
     ZG_REQUIRE((!vfreq || V % 2 == 0) && rot.dims % 2 == 0 && rot.dims <= D, ZG_ERR_ARG, "windowed attention: %d value channels, %d of %d rotated", V, rot.dims, D);
-    window_prep_kernel<<<M, 256, 0, s>>>(proj, ld, H, G, D, V, rot, vfreq, row_pos, row_slot, page_table, max_pages, page_tokens, cache);
+    window_prep_kernel<<<M, 256, 0, s>>>(proj, ld, H, G, D, V, rot, vfreq, row_pos, row_slot, page_table, max_pages, page_tokens, cache, vals);
     ZG_HIP(hipGetLastError());
     return ZG_OK;
 }
@@ -1398,7 +1423,7 @@ int launch_window_attention_split(const float* q, int ldq, float* out, int ldo, 
                                   size_t ws_floats, const int* ent_start, const int* ent_len, int n_entries, hipStream_t s, bool* taken,
                                   const float* out_gate, int ld_gate, float out_factor, ScoreShape shape) {
     *taken = false;
-    if (M <= 0) return ZG_OK;
+    if (M <= 0 || shape.gate) return ZG_OK;  // (weights that need no statistics: launch_gate_attention)
     if (mask.window <= 0) mask.keep = 0;
     if (const char* e = getenv("ZGPT2_LM_WINDOW_GENERAL"))  // test hook: every step through the general kernel
         if (atoi(e) != 0) return ZG_OK;

@@ -160,10 +160,11 @@ typedef std::vector<std::pair<std::string, std::vector<float>>> DerivedTensors;
 inline void build_config(const Json& cfg, const Json* tensors, std::vector<zg_lm_layer>& layers, zg_lm_config& out, DerivedTensors* derived = nullptr) {
     const Json* arch = cfg.get("architecture");
     const std::string design = arch ? arch->str : std::string("?");
-    if (design != "Tokosun" && design != "Gupizen" && design != "Sanazen" && design != "Vovalorn" && design != "Duvulix")
+    if (design != "Tokosun" && design != "Gupizen" && design != "Sanazen" && design != "Vovalorn" && design != "Duvulix" && design != "Pemuvik")
         throw std::runtime_error("config: architecture '" + design + "' is not served");
-    const bool gup = design == "Gupizen", san = design == "Sanazen", vov = design == "Vovalorn", duv = design == "Duvulix";
+    const bool gup = design == "Gupizen", san = design == "Sanazen", vov = design == "Vovalorn", duv = design == "Duvulix", pem = design == "Pemuvik";
     memset(&out, 0, sizeof(out));
+    if (pem) out.flags |= ZG_LM_SIDE_BY_SIDE | ZG_LM_LAYER_SCALE | ZG_LM_TIED_HEAD;  // what the name fixes
     if (duv) out.flags |= ZG_LM_NO_SHIFT;  // what the name fixes: the mixer reads the norm as it is
     if (vov) {  // what the name fixes: norms without statistics, one of them behind the embedding
         out.flags |= ZG_LM_TANH_NORMS | ZG_LM_EMBED_NORM;
@@ -226,6 +227,10 @@ inline void build_config(const Json& cfg, const Json* tensors, std::vector<zg_lm
         d.dim = (int)sizes.at(duv && type == "mamba2" ? "state" : "dim").num;
         d.vdim = sizes.get("vdim") ? (int)sizes.at("vdim").num : d.dim;
         if (duv) d.rot_halves = 1;
+        if (pem) {
+            d.ff_act = ZG_LM_ACT_GLU_SILU;
+            d.router = ZG_LM_ROUTE_SOFTMAX_GROUPS;
+        }
         auto yarn_rotary = [&] {
             d.rot_base = 10000.0f;
             const Json* rot = m.get("rot");
@@ -339,6 +344,18 @@ inline void build_config(const Json& cfg, const Json* tensors, std::vector<zg_lm
             if (const Json* v = m.get("dist_bias")) d.dist_bias = v->truthy() ? 1 : 0;
         } else if (vov) {
             throw std::runtime_error("config: unknown mixer type '" + type + "'");
+        } else if (pem && type == "attention") {
+            d.mixer = ZG_LM_MIX_ROTARY_ATTENTION;
+            d.kv_heads = m.get("kv_heads") ? (int)m.at("kv_heads").num : d.heads;
+            d.scale = (float)m.at("scale").num;
+            d.proj_bias = d.value_norm = d.sigmoid_weights = 1;
+            if (const Json* v = m.get("v_mix")) d.value_mix = v->truthy() ? 1 : 0;
+            if (const Json* mask = m.get("mask"))
+                if (mask->truthy())
+                    if (const Json* v = mask->get("size")) d.window = (int)v->num;
+            yarn_rotary();
+        } else if (pem && type != "latent_attention") {
+            throw std::runtime_error("config: unknown mixer type '" + type + "'");
         } else if (duv && type == "attention") {
             d.mixer = ZG_LM_MIX_ROTARY_ATTENTION;
             d.kv_heads = m.get("kv_heads") ? (int)m.at("kv_heads").num : d.heads;
@@ -364,6 +381,8 @@ inline void build_config(const Json& cfg, const Json* tensors, std::vector<zg_lm
                 d.head_gate = 1;
                 if (const Json* v = m.get("kv_from"))
                     if (v->kind == Json::Num) d.kv_from = (int)v->num + 1;
+            } else if (pem) {  // queries projected directly, a sink per head
+                d.sink = 1;
             } else {
                 d.q_rank = (int)m.at("q_rank").num;
             }
@@ -380,6 +399,7 @@ inline void build_config(const Json& cfg, const Json* tensors, std::vector<zg_lm
                 d.ff = ZG_LM_FF_DENSE;
                 d.ff_width = (int)mlp->at("ff").num;
                 if (duv) d.dense_act = ZG_LM_DENSE_POLYNORM;
+                if (pem) d.dense_act = ZG_LM_DENSE_GLU_GELU;
             } else if (kind == "moe") {
                 d.ff = ZG_LM_FF_MOE;
                 d.ff_width = (int)mlp->at("expert").at("ff").num;
@@ -393,7 +413,13 @@ inline void build_config(const Json& cfg, const Json* tensors, std::vector<zg_lm
                         d.shared_limit = (float)sh->at("limit").num;
                     }
                 }
-                if (vov) {
+                if (pem) {
+                    const Json* sh = mlp->get("shared");
+                    d.shared_gate = sh && sh->truthy() ? 1 : 0;
+                    if (const Json* v = mlp->at("router").get("identity"))
+                        if (v->truthy()) d.identity = (int)v->num;
+                }
+                if (vov || pem) {
                     const Json& r = mlp->at("router");
                     d.route_groups = d.route_keep = 1;
                     d.route_scale = r.get("scale") ? (float)r.at("scale").num : 1.0f;

@@ -34,6 +34,13 @@ config.json (zig_gpt2_amd/models.py maps architecture names to loaders; `DESIGNS
   kv_from: j: the layer reads layer j's latents instead of making its own) | "attention" (grouped-query attention, rotary with
   YaRN scaling; a query sees its own chunk of mask.size positions) | "mamba2" (selective state space: heads, vdim, state, groups,
   conv, norm_groups); the mixer reads norm1(x) as it is; dense feed-forwards with a polynomial activation (tensor mlp.act).
+  Pemuvik: type "latent_attention" (queries projected directly, neighbouring rotary pairs, the softmax's denominator with a sink per
+  head) | "attention" (grouped-query attention in a window of mask.size positions whose weights are sigmoid(score + pb[h]), nothing
+  normalised over the keys; biases on all projections; every value head divided by its root mean square; v_mix: the first such
+  layer's values of the same token mixed in by the scalar vmix); a layer is x += ls1 * mixer(norm1(x)) + ls2 * mlp(norm2(x)) with
+  plain norm weights; dense feed-forwards gated by gelu; experts chosen by softmax scores + correction among the best contiguous
+  blocks of router outputs (a block ranks by its largest), the last router.identity outputs standing for the input itself,
+  weights normalised over the chosen; mlp.shared: an expert every token uses, times sigmoid(shared.sg . h); tied head.
 """
 import ctypes as C
 import json
@@ -49,11 +56,11 @@ from ._lib import check_lm as check
 MIXERS = {"hgrn2": _lib.LM_MIX_HGRN2, "latent_attention": _lib.LM_MIX_LATENT_ATTENTION, "parallel": _lib.LM_MIX_PARALLEL,
           "channel_delta": _lib.LM_MIX_CHANNEL_DELTA, "window_linear": _lib.LM_MIX_WINDOW_LINEAR, "gla": _lib.LM_MIX_GLA,
           "attention": _lib.LM_MIX_ATTENTION, "rotary_attention": _lib.LM_MIX_ROTARY_ATTENTION, "ssd": _lib.LM_MIX_SSD}
-DENSE_ACTS = {"relu2": _lib.LM_DENSE_RELU2, "polynorm": _lib.LM_DENSE_POLYNORM}
+DENSE_ACTS = {"relu2": _lib.LM_DENSE_RELU2, "polynorm": _lib.LM_DENSE_POLYNORM, "glu_gelu": _lib.LM_DENSE_GLU_GELU}
 ROT_STYLES = {"yarn": _lib.LM_ROT_YARN, "bands": _lib.LM_ROT_BANDS}
 EXPERT_ACTS = {"glu_silu": _lib.LM_ACT_GLU_SILU, "gelu": _lib.LM_ACT_GELU, "glu_clipped": _lib.LM_ACT_GLU_CLIPPED}
 ROUTERS = {"softmax_all": _lib.LM_ROUTE_SOFTMAX_ALL, "top_logits": _lib.LM_ROUTE_TOP_LOGITS, "sigmoid_input": _lib.LM_ROUTE_SIGMOID_INPUT,
-           "sigmoid_groups": _lib.LM_ROUTE_SIGMOID_GROUPS}
+           "sigmoid_groups": _lib.LM_ROUTE_SIGMOID_GROUPS, "softmax_groups": _lib.LM_ROUTE_SOFTMAX_GROUPS}
 
 # what an architecture name fixes beyond config.json.  mixers: layer type of config.json -> mixer of the library (two designs
 # call different pairs of branches "parallel")
@@ -67,7 +74,11 @@ DESIGNS = {
     "Vovalorn": dict(mixers={"gla": "gla", "attention": "attention"}, tied_head=False, loop_readd=False, expert_act="glu_silu", router="sigmoid_groups",
                      tanh_norms=True, embed_norm=True),
     "Duvulix": dict(mixers={"latent_attention": "latent_attention", "attention": "rotary_attention", "mamba2": "ssd"}, tied_head=False, loop_readd=False,
-                    expert_act="glu_silu", router="softmax_all", no_shift=True, dense_act="polynorm", rot_halves=True, direct_queries=True),
+                    expert_act="glu_silu", router="softmax_all", no_shift=True, dense_act="polynorm", rot_halves=True, direct_queries=True,
+                    latent=dict(head_gate=True), attention=dict(mask="chunk")),
+    "Pemuvik": dict(mixers={"latent_attention": "latent_attention", "attention": "rotary_attention"}, tied_head=True, loop_readd=False, expert_act="glu_silu",
+                    router="softmax_groups", side_by_side=True, layer_scale=True, dense_act="glu_gelu", direct_queries=True, shared_gate=True,
+                    latent=dict(sink=True), attention=dict(mask="window", proj_bias=True, value_norm=True, sigmoid_weights=True)),
 }
 
 
@@ -126,6 +137,13 @@ class LayerSpec:
     head_gate: bool = False  # latent attention: head h times sigmoid(W_g h)_h
     norm_groups: int = 0  # ssd: parts of the norm behind the gate (ssd: dim = state rows, kv_heads = groups of B and C)
     dense_act: str = "relu2"
+    proj_bias: bool = False  # rotary attention: biases on q, k, v and o
+    value_norm: bool = False  # rotary attention: every value head divided by its root mean square
+    value_mix: bool = False  # rotary attention: the first such layer's values mixed in
+    sigmoid_weights: bool = False  # rotary attention: a key weighs sigmoid(score + pb[h]), no softmax
+    sink: bool = False  # latent attention: exp(sink[h]) in the softmax's denominator
+    identity: int = 0  # softmax_groups: router outputs behind the experts that stand for the input itself
+    shared_gate: bool = False  # glu_silu: the shared expert times sigmoid(shared.sg . h)
 
     @classmethod
     def from_json(cls, entry, design="Tokosun", shapes=None, prefix=""):
@@ -178,9 +196,10 @@ class LayerSpec:
             kw = dict(mixer=kind, heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=int(m["dim"]), vdim=int(m["vdim"]),
                       conv=int(m["conv"]), decay_rank=inner("decay_rank", "mix.a1"), gate_rank=inner("gate_rank", "mix.g1"))
         elif kind == "rotary_attention":
-            rot = m.get("rot") or {}
+            rot, att = m.get("rot") or {}, dict(fixed["attention"])
+            size = {att.pop("mask"): int((m.get("mask") or {}).get("size", 0))}  # the design's mask: a window or chunks of this size
             kw = dict(mixer=kind, heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=int(m["dim"]),
-                      vdim=int(m.get("vdim", m["dim"])), scale=float(m["scale"]), chunk=int((m.get("mask") or {}).get("size", 0)),
+                      vdim=int(m.get("vdim", m["dim"])), scale=float(m["scale"]), value_mix=bool(m.get("v_mix", False)), **size, **att,
                       rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 10000.0)),
                       rot_scaling=dict(rot["scaling"]) if rot.get("scaling") else None)
         elif kind == "ssd":
@@ -193,7 +212,7 @@ class LayerSpec:
         if kind == "latent_attention":
             rot = m.get("rot") or {}
             direct = bool(fixed.get("direct_queries"))
-            kw.update(head_gate=direct, kv_from=int(m["kv_from"]) if m.get("kv_from") is not None else None)
+            kw.update(**fixed.get("latent", {}), kv_from=int(m["kv_from"]) if m.get("kv_from") is not None else None)
             kw.update(rot_dim=int(m["rot_dim"]), kv_rank=int(m["kv_rank"]), q_rank=0 if direct else int(m["q_rank"]), scale=float(m["scale"]),
                       rot_dims=int(rot.get("dims", m["rot_dim"])), rot_base=float(rot.get("base", 10000.0)),
                       rot_scaling=dict(rot["scaling"]) if rot.get("scaling") else None)
@@ -208,8 +227,10 @@ class LayerSpec:
                     if mlp.get("shared"):
                         kw.update(shared_width=int(mlp["shared"]["ff"]), shared_limit=float(mlp["shared"]["limit"]))
                 elif mlp.get("shared"):
-                    kw.update(shared_width=int(mlp["shared"]["ff"]))
-                if fixed["router"] == "sigmoid_groups":
+                    kw.update(shared_width=int(mlp["shared"]["ff"]), shared_gate=bool(fixed.get("shared_gate")))
+                if fixed["router"] == "softmax_groups":
+                    kw.update(identity=int(mlp["router"].get("identity") or 0))
+                if fixed["router"] in ("sigmoid_groups", "softmax_groups"):
                     groups = mlp["router"].get("groups") or {}
                     count = int(groups.get("count", 1))
                     kw.update(route_groups=count, route_keep=int(groups.get("keep", count)), route_scale=float(mlp["router"].get("scale", 1.0)))
@@ -252,8 +273,10 @@ class LayerSpec:
                 mixer["rot"] = {"base": self.rot_base, "dims": self.rot_dims}
                 if self.rot_scaling:
                     mixer["rot"]["scaling"] = dict(self.rot_scaling)
-            if self.chunk:
-                mixer["mask"] = {"size": self.chunk}
+            if self.chunk or self.window:
+                mixer["mask"] = {"size": self.chunk or self.window}
+            if self.value_mix:
+                mixer["v_mix"] = True
         elif self.mixer == "ssd":
             mixer = {"heads": self.heads, "vdim": self.vdim, "state": self.dim, "groups": self.kv_heads, "conv": self.conv, "norm_groups": self.norm_groups}
         if self.mixer == "gla":
@@ -278,6 +301,11 @@ class LayerSpec:
                 mlp["shared"] = {"ff": self.shared_width}
             if self.router == "sigmoid_groups":
                 mlp["router"].update(groups={"count": self.route_groups, "keep": self.route_keep}, scale=self.route_scale)
+            elif self.router == "softmax_groups":
+                if self.route_groups > 1:
+                    mlp["router"]["groups"] = {"count": self.route_groups, "keep": self.route_keep}
+                if self.identity:
+                    mlp["router"]["identity"] = self.identity
         kinds = {"window_linear": "parallel", "rotary_attention": "attention", "ssd": "mamba2"}  # config.json's names where they differ
         out = {"type": kinds.get(self.mixer, self.mixer), "mixer": mixer, "mlp": mlp}
         if self.weights_of is not None:
@@ -297,16 +325,20 @@ class LayerSpec:
                             self.lin_heads, self.lin_dim, self.lin_vdim, self.ff_limit, self.shared_width, self.shared_limit, self.tau, self.softcap,
                             self.qtemp_coef, self.qtemp_every, int(self.dist_bias), self.route_groups, self.route_keep, self.route_scale,
                             0 if self.weights_of is None else self.weights_of + 1, int(self.rot_halves), self.chunk,
-                            0 if self.kv_from is None else self.kv_from + 1, int(self.head_gate), self.norm_groups, DENSE_ACTS[self.dense_act])
+                            0 if self.kv_from is None else self.kv_from + 1, int(self.head_gate), self.norm_groups, DENSE_ACTS[self.dense_act],
+                            int(self.proj_bias), int(self.value_norm), int(self.value_mix), int(self.sigmoid_weights), int(self.sink), self.identity,
+                            int(self.shared_gate))
 
-    def tensor_shapes(self, prefix, width, canon_taps=0, tanh_norms=False, no_shift=False):
+    def tensor_shapes(self, prefix, width, canon_taps=0, tanh_norms=False, no_shift=False, side=False, layer_scale=False):
         """{checkpoint tensor name: shape} of this layer (none for a layer that runs another layer's tensors)."""
         if self.weights_of is not None:
             return {}
         H, D, V, W = self.heads, self.dim, self.vdim, width
         t = {prefix + "norm1": (W,), prefix + "norm1b": (W,)}
-        if self.mixer == "window_linear":  # plain norms in front of the sublayers only, nothing between norm and mixer
+        if side:  # plain norms in front of the sublayers only, nothing between norm and mixer
             t = {prefix + "norm1": (W,)}
+            if layer_scale:
+                t.update({prefix + n: (W,) for n in (("ls1", "ls2") if self.ff != "none" else ("ls1",))})
         elif tanh_norms or no_shift:  # the mixer reads the norm as it is
             pass
         elif canon_taps:
@@ -359,8 +391,16 @@ class LayerSpec:
             t.update({m + "uk": (H * D, KR), m + "uv": (H * V, KR), m + "o": (W, H * V)})
             if self.head_gate:
                 t[m + "g"] = (H, W)
+            if self.sink:
+                t[m + "sink"] = (H,)
         elif self.mixer == "rotary_attention":
             t.update({m + "q": (H * D, W), m + "k": (self.kv_heads * D, W), m + "v": (self.kv_heads * V, W), m + "o": (W, H * V)})
+            if self.proj_bias:
+                t.update({m + n + ".b": (t[m + n][0],) for n in ("q", "k", "v", "o")})
+            if self.sigmoid_weights:
+                t[m + "pb"] = (H,)
+            if self.value_mix:
+                t[m + "vmix"] = ()
         elif self.mixer == "ssd":
             inner, bc = H * V, 2 * self.kv_heads * D
             t.update({m + "in": (2 * inner + bc + H, W), m + "conv": (inner + bc, self.conv), m + "conv.b": (inner + bc,), m + "dt_bias": (H,),
@@ -368,24 +408,26 @@ class LayerSpec:
         f = prefix + "mlp."
         if self.ff != "none":
             t.update({prefix + "norm2": (W,), prefix + "norm2b": (W,)})
-            if self.mixer == "window_linear":
+            if side:
                 del t[prefix + "norm2b"]
         if self.ff == "dense":
             t.update({f + "up": (self.ff_width, W), f + "down": (W, self.ff_width)})
             if self.dense_act == "polynorm":
                 t[f + "act"] = (4,)
+            elif self.dense_act == "glu_gelu":
+                t[f + "gate"] = (self.ff_width, W)
         elif self.ff == "moe":
             for e in range(self.experts):
                 t.update({f"{f}e{e}.up": (self.ff_width, W), f"{f}e{e}.down": (W, self.ff_width)})
                 if self.expert_act in ("glu_silu", "glu_clipped"):
                     t[f"{f}e{e}.gate"] = (self.ff_width, W)
-            t[f + "router"] = (self.experts, W)
+            t[f + "router"] = (self.experts + self.identity, W)
             if self.router != "sigmoid_input":
-                t[f + ("router.b" if self.router == "top_logits" else "correction")] = (self.experts,)
+                t[f + ("router.b" if self.router == "top_logits" else "correction")] = (self.experts + self.identity,)
             if self.shared_width:
                 S = self.shared_width
                 t.update({f + "shared.gate": (S, W), f + "shared.up": (S, W), f + "shared.down": (W, S)})
-                if self.expert_act == "glu_clipped":
+                if self.expert_act == "glu_clipped" or self.shared_gate:
                     t[f + "shared.sg"] = (1, W)
         if tanh_norms:  # every norm's bias and scalar beside its weight
             for name in [k for k in t if k[len(prefix):] in ("norm1", "norm1b", "norm2", "norm2b")]:
@@ -461,7 +503,7 @@ class LMConfig:
             out["logit_softcap"] = self.logit_softcap
         if self.residual_mult != 1.0:
             out["residual_mult"] = self.residual_mult
-        if out["loop"] is None and (DESIGNS[self.architecture].get("tanh_norms") or DESIGNS[self.architecture].get("no_shift")):
+        if out["loop"] is None and any(DESIGNS[self.architecture].get(k) for k in ("tanh_norms", "no_shift", "layer_scale")):
             del out["loop"]
         return out
 
@@ -474,7 +516,7 @@ class LMConfig:
         return ((_lib.LM_TIED_HEAD if d["tied_head"] else 0) | (_lib.LM_LOOP_READD if d["loop_readd"] else 0) |
                 (_lib.LM_SIDE_BY_SIDE if d.get("side_by_side") else 0) | (_lib.LM_SINUSOID_POSITIONS if d.get("sinusoid_positions") else 0) |
                 (_lib.LM_TANH_NORMS if d.get("tanh_norms") else 0) | (_lib.LM_EMBED_NORM if d.get("embed_norm") else 0) |
-                (_lib.LM_NO_SHIFT if d.get("no_shift") else 0))
+                (_lib.LM_NO_SHIFT if d.get("no_shift") else 0) | (_lib.LM_LAYER_SCALE if d.get("layer_scale") else 0))
 
     def passes(self):
         """Layer index of every pass, in execution order."""
@@ -495,7 +537,8 @@ class LMConfig:
         if not self.tied_head:
             t["head"] = (self.vocab, self.width)
         for i, l in enumerate(self.layers):
-            t.update(l.tensor_shapes(f"l{i}.", self.width, self.canon_taps, tanh_norms, bool(d.get("no_shift"))))
+            t.update(l.tensor_shapes(f"l{i}.", self.width, self.canon_taps, tanh_norms, bool(d.get("no_shift")), bool(d.get("side_by_side")),
+                                     bool(d.get("layer_scale"))))
         return t
 
     def derived_tensors(self):

@@ -56,6 +56,13 @@ def _load_duvulix(path, dtype="bfloat16", **kw):
     return lm.LayeredLM.from_dir(path, dtype=dtype, **kw)
 
 
+@register("Pemuvik")
+def _load_pemuvik(path, dtype="bfloat16", **kw):
+    from . import lm
+
+    return lm.LayeredLM.from_dir(path, dtype=dtype, **kw)
+
+
 @register("gpt2")
 def _load_gpt2(path, dtype="float32", config="124M", **kw):
     from . import gpt
