@@ -299,9 +299,10 @@ __global__ __launch_bounds__(256, NKS <= 8 ? 2 : 1) void gate_tiles_kernel(const
 #pragma unroll
         for (int i = 0; i < 16; ++i) o[t][i] = 0.0f;
 
-    const int kt_lo = first_key(pos0, a.mask) / 32, kt_hi = last / 32;
+    const int blk_first = first_key(pos0, a.mask), kt_lo = blk_first / 32, kt_hi = last / 32;
     for (int kt = kt_lo + wave; kt <= kt_hi; kt += 4) {
-        const int j = min(32 * kt + r, last);  // (positions behind the block's last row hold nothing yet)
+        // (positions behind the block's last row hold nothing yet, those in front of its first row's keys perhaps nothing any more)
+        const int j = min(max(32 * kt + r, blk_first), last);
         const int crow = cache_row(pages, j, a.page_tokens, a.max_pages);
         const float* kp = a.cache + (size_t)crow * cstride + (size_t)g * D;
         f32x16 sc;
