@@ -48,11 +48,12 @@ def parse():
                    help="instead of the default workload: prompt and decode throughput of a layered model (Tokosun design, random weights) "
                         "at a size that resembles GPT-2 124M / medium / XL, beside the GPT-2 model of the same width and depth")
     p.add_argument("--lm-dtype", default="bfloat16", choices=["bfloat16", "float32"])
-    p.add_argument("--lm-design", default="tokosun", choices=["tokosun", "gupizen", "sanazen", "vovalorn", "duvulix"],
+    p.add_argument("--lm-design", default="tokosun", choices=["tokosun", "gupizen", "sanazen", "vovalorn", "duvulix", "pemuvik"],
                    help="with --lm: which design is measured.  gupizen: a Gupizen stack of the same width and depth, beside the Tokosun stack "
                         "(the tier's closest model) instead of GPT-2.  sanazen: a Sanazen stack beside the Gupizen stack of the same width and depth.  "
                         "vovalorn: a Vovalorn stack beside the Tokosun stack of the same width and depth; "
-                        "duvulix: a Duvulix stack beside the Tokosun stack of the same width and depth")
+                        "duvulix: a Duvulix stack beside the Tokosun stack of the same width and depth; "
+                        "pemuvik: a Pemuvik stack beside the Duvulix stack of the same width and depth")
     p.add_argument("--dry-run", action="store_true",
                    help="CPU rehearsal of the launch path (gloo, no GPU, no kernels): rendezvous, prompt sharding, "
                         "weight-arena broadcast, barriers and the max-reduce; prints a line with dry_run=true")
@@ -524,17 +525,38 @@ def duvulix_bench_config(width, n_layers, vocab, chunk=512):
     return lm.LMConfig(vocab=vocab, width=width, layers=layers, norm_eps=1e-6, architecture="Duvulix")
 
 
+def pemuvik_bench_config(width, n_layers, vocab, window=512):
+    """A Pemuvik-design stack of `n_layers` layers in the repeating order windowed attention + dense, windowed attention + experts, windowed
+    attention + dense, latent attention + experts: attention heads of 64 channels on a quarter (a fifth) as many key heads in a
+    window of `window` tokens, half of the channels rotated, values mixed in every attention layer; latent heads of 64 + 32
+    channels on latents of 256 with sinks; dense feed-forwards of 3 x width (gated), 8 experts of width `width` in 2 groups of 5
+    router outputs (2 of them pass through) of which one stays and 2 outputs are chosen, and a shared expert of the same width."""
+    from zig_gpt2_amd import lm
+
+    heads = width // 64
+    kv = heads // 4 if heads % 4 == 0 else heads // 5 if heads % 5 == 0 else heads
+    dense = dict(ff="dense", ff_width=3 * width, dense_act="glu_gelu")
+    moe = dict(ff="moe", ff_width=width, experts=8, top=2, expert_act="glu_silu", router="softmax_groups", route_groups=2, route_keep=1, identity=2,
+               shared_width=width, shared_gate=True)
+    att = dict(mixer="rotary_attention", heads=heads, kv_heads=kv, dim=64, vdim=64, scale=64 ** -0.5, window=window, rot_dims=32, rot_base=10000.0,
+               proj_bias=True, value_norm=True, value_mix=True, sigmoid_weights=True)
+    lat = dict(mixer="latent_attention", heads=heads, dim=64, vdim=64, rot_dim=32, kv_rank=256, scale=(64 + 32) ** -0.5, rot_dims=32, rot_base=10000.0,
+               sink=True)
+    order = [dict(att, **dense), dict(att, **moe), dict(att, **dense), dict(lat, **moe)]
+    return lm.LMConfig(vocab=vocab, width=width, layers=[lm.LayerSpec(**order[i % 4]) for i in range(n_layers)], norm_eps=1e-6, architecture="Pemuvik")
+
+
 def lm_weight_bytes(cfg):
     """(stored, read per decoded token) bytes of the bf16 matrices: every expert is stored, `top` of them are read."""
     stored = active = 0
     for name, shape in cfg.tensor_shapes().items():
-        if len(shape) != 2 or name == "embed":
+        if len(shape) != 2 or (name == "embed" and not cfg.tied_head):
             continue
         b = 2 * shape[0] * shape[1]
         stored += b
         if ".mlp.e" in name:
             lay = cfg.layers[int(name[1:name.index(".")])]
-            b = b * lay.top / lay.experts
+            b = b * lay.top / (lay.experts + lay.identity)
         active += b
     return int(stored), int(active)
 
@@ -552,6 +574,7 @@ def lm_bench(a):
     san = a.lm_design == "sanazen"
     vov = a.lm_design == "vovalorn"
     duv = a.lm_design == "duvulix"
+    pem = a.lm_design == "pemuvik"
     cfg = lm_bench_config(width, n_layers, gcfg.vocab_size)
     out = {"metric": "lm_decode_tokens_per_s", "unit": "tokens/s", "n_gpus": 1, "steps": a.steps, "warmup": a.warmup, "higher_is_better": True,
            "scaling": "weak", "vs_baseline": None, "dtype": "bf16" if a.lm_dtype == "bfloat16" else "fp32", "data": "synthetic (random weights, filled on the GPU)",
@@ -629,6 +652,15 @@ def lm_bench(a):
         out["config"]["model"] = (f"Duvulix design, width {width}, {n_layers} layers (state space, latent attention, latent attention on the same "
                                   f"latents, attention in chunks of 512; dense feed-forwards), vocab {gcfg.vocab_size}")
         out.update(value=d1["tokens_per_s"], ms_per_step=round(d1["wall_us_per_step"] / 1e3, 4), duvulix=d_res, tokosun_equal_size=t_res)
+        print(json.dumps(out))
+        return
+    if pem:  # beside the tier's closest model (rotary grouped-query attention in pieces of 512 positions, latent attention with direct queries)
+        p_res = measure(pemuvik_bench_config(width, n_layers, gcfg.vocab_size))
+        d_res = measure(duvulix_bench_config(width, n_layers, gcfg.vocab_size))
+        d1 = p_res["decode"][0]
+        out["config"]["model"] = (f"Pemuvik design, width {width}, {n_layers} layers (sigmoid-weight attention in a window of 512 + dense, the same + experts, "
+                                  f"the same + dense, latent attention with sinks + experts; 8 experts and 2 pass-through outputs, 2 chosen, one shared), vocab {gcfg.vocab_size}")
+        out.update(value=d1["tokens_per_s"], ms_per_step=round(d1["wall_us_per_step"] / 1e3, 4), pemuvik=p_res, duvulix_equal_size=d_res)
         print(json.dumps(out))
         return
     if gup:  # the new design beside the tier's closest model at equal width and depth
