@@ -173,6 +173,29 @@ def test_decode_batches_of_every_size():
     m.close()
 
 
+def test_decode_batches_of_many_heads():
+    """Eight rows of 90 heads, five to a key head: a workgroup of the decode kernel then takes four query heads of a key head (and the fifth
+    alone) instead of one; heads of each of the kernel's sizes, decoded in lock step and in steps of two entries with two to four rows."""
+    cfg = pl.config([pl.attn_layer(heads=90, kv_heads=18, dim=6, vdim=5, size=20, v_mix=False), pl.attn_layer(heads=65, kv_heads=13, dim=70, vdim=9, scale=0.1, size=0, v_mix=False),
+                     pl.attn_layer(heads=70, kv_heads=10, dim=9, vdim=130, size=11, v_mix=False)], width=20)
+    w = pl.weights(cfg, seed=25)
+    m = make(cfg, w, max_seqs=8, page_tokens=8)
+    seqs = [pl.tokens(120 + i, 12 + 5 * i + 8, cfg["vocab"]) for i in range(8)]
+    refs = [po.forward(w, cfg, t) for t in seqs]
+    slots = [m.open() for _ in seqs]
+    at = [12 + 5 * i for i in range(8)]
+    m.step([(s, t[:k], []) for s, t, k in zip(slots, seqs, at)])
+    for counts in ([1] * 8, [1] * 8, [4, 4], [2, 3], [1] * 8):
+        got = m.step([(slots[i], seqs[i][at[i]:at[i] + c], list(range(c))) for i, c in enumerate(counts) if at[i] + c <= len(seqs[i])])
+        off = 0
+        for i, c in enumerate(counts):
+            if at[i] + c <= len(seqs[i]):
+                tl.assert_close(got[off:off + c], refs[i][at[i]:at[i] + c], "float32", (counts, i))
+                off += c
+                at[i] += c
+    m.close()
+
+
 def test_slots_and_pages_are_reused():
     """Two slots and a cache of 96 tokens in pages of 4.  A closed sequence gives its pages and its slot back; the next one starts on pages
     that held other keys, values and latents."""

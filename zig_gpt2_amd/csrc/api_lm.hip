@@ -929,14 +929,18 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
         const int all_keys = g->max_pages * g->P;
         return replayed ? (g->bucket_keys > 0 ? g->bucket_keys : all_keys) : std::min(all_keys, (g->step_keys + 63) / 64 * 64);
     };
-    // the dense feed-forward of a layer: in -> out
-    auto dense_ff = [&](const LayerW& L, const float* in, float* out) -> int {
+    // the dense feed-forward of a layer: in -> out (first_done: its first product has been launched)
+    auto dense_up = [&](const LayerW& L, const float* in) {
+        Linear up;
+        up.A = in; up.lda = W; up.B = L.up; up.ldb = W; up.C = g->u; up.ldc = L.n_up; up.M = M; up.N = L.n_up; up.K = W;
+        up.act = L.d.dense_act == ZG_LM_DENSE_RELU2 ? ACT_RELU2 : ACT_NONE;
+        return up;
+    };
+    auto dense_ff = [&](const LayerW& L, const float* in, float* out, bool first_done = false) -> int {
         const int F = L.d.ff_width;
         const bool poly = L.d.dense_act == ZG_LM_DENSE_POLYNORM, gated = L.d.dense_act == ZG_LM_DENSE_GLU_GELU;
-        Linear up, dn;
-        up.A = in; up.lda = W; up.B = L.up; up.ldb = W; up.C = g->u; up.ldc = L.n_up; up.M = M; up.N = L.n_up; up.K = W;
-        up.act = poly || gated ? ACT_NONE : ACT_RELU2;
-        ZG_TRY(launch_linear(up, f32, s));
+        Linear dn;
+        if (!first_done) ZG_TRY(launch_linear(dense_up(L, in), f32, s));
         if (gated) {  // rows gate | up
             dn.B = L.down; dn.ldb = F; dn.C = out; dn.ldc = W; dn.M = M; dn.N = W; dn.K = F;
             if (M <= 2) {  // the activation where the second product reads its rows (more rows: every workgroup would redo it)
@@ -955,6 +959,13 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
         }
         dn.A = g->u; dn.lda = F; dn.B = L.down; dn.ldb = F; dn.C = out; dn.ldc = W; dn.M = M; dn.N = W; dn.K = F;
         return launch_linear(dn, f32, s);
+    };
+    // one-row steps of side-by-side sublayers: the dense feed-forward's first product rides in the launch of the mixer's first
+    const LayerW* up_done = nullptr;
+    auto first_product = [&](const LayerW& L, const Linear& lin) -> int {
+        if (!(side && M == 1 && L.d.ff == ZG_LM_FF_DENSE)) return launch_linear(lin, f32, s);
+        up_done = &L;
+        return launch_linear_pair(lin, dense_up(L, g->hc), f32, s);
     };
     bool h_ready = false;  // g->h already holds this pass's shifted norm (written by the previous pass's fused tail)
     if (tnorm) {  // the norm behind the embedding (in place) and the first pass's norm; every later one rides behind a sublayer's sum
@@ -1008,7 +1019,7 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             mask.chunk = d.chunk;
             lin.A = hin; lin.lda = W; lin.B = L.wcat; lin.ldb = W; lin.C = g->proj; lin.ldc = LD; lin.M = M; lin.N = L.n_cat; lin.K = W;
             lin.bias = L.qkv_bias;
-            ZG_TRY(launch_linear(lin, f32, s));
+            ZG_TRY(first_product(L, lin));
             ValuePrep vals;
             vals.norm = d.value_norm != 0;
             vals.eps = eps;
@@ -1216,7 +1227,7 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             const Rotary rot{L.rot_freq, d.rot_dims, L.rot_amp, d.rot_halves};
             lin = Linear();
             lin.A = hin; lin.lda = W; lin.B = L.dqkv; lin.ldb = W; lin.C = g->proj; lin.ldc = LD; lin.M = M; lin.N = L.n_cat; lin.K = W;
-            ZG_TRY(launch_linear(lin, f32, s));
+            ZG_TRY(first_product(L, lin));
             const float* gate = d.head_gate ? g->proj + L.n_cat - H : nullptr;
             const float* q = direct ? g->proj : g->q;
             const int ldq = direct ? LD : H * (D + R);
@@ -1339,7 +1350,8 @@ int enqueue_layers(zg_lm* g, int M, int n_ent, bool capturing, bool single) {
             const int F = d.ff_width;
             const float* fin = g->hc;
             if (d.ff == ZG_LM_FF_DENSE) {
-                ZG_TRY(dense_ff(L, fin, g->y2));
+                ZG_TRY(dense_ff(L, fin, g->y2, up_done == &L));
+                up_done = nullptr;
             } else if (d.ff == ZG_LM_FF_MOE) {
                 const int E = d.experts, top = d.top, NA = M * top;
                 const int UF = d.ff_act == ZG_LM_ACT_GELU ? F : 2 * F;

@@ -2,7 +2,8 @@
 // the keys.  A row's result is a plain sum, so shares of its keys add up in any grouping and no pass over the scores is needed in
 // front of the values:
 //   * gate_rows_kernel    steps of few rows (decode): a workgroup of sixteen waves per (share of the keys, row, key head), eight keys to a
-//                         wave and trip, up to kGateHeads query heads of the key head on every key read.  Steps of one row per entry
+//                         wave and trip, up to four query heads of the key head on every key read (one, while there are few rows and heads:
+//                         a compute unit is then busy with the weights and sums of its heads, not with its loads).  Steps of one row per entry
 //                         also prepare the row here — rotary q and k, the value's norm and mix, the token's cache row.
 //   * gate_tiles_kernel   prompt portions: 32 consecutive rows of an entry and one head per workgroup, tiles of 32 keys dealt to the four
 //                         waves; both products on the matrix cores, operands straight from the cache rows to registers.
@@ -47,7 +48,6 @@ struct GateArgs {
 // ------------------------------------------------------------------------------------------------ few rows
 constexpr int kGateWaves = 16;
 constexpr int kGateKeys = 8;   // keys of a wave per trip: eight lanes share a key's channels
-constexpr int kGateHeads = 4;  // query heads of one key head per workgroup
 
 // channel i of a vector of rot.dims turned channels at position pos
 __device__ __forceinline__ float rotary_at(const float* v, int i, float fpos, const Rotary& rot) {
@@ -60,18 +60,19 @@ __device__ __forceinline__ float rotary_at(const float* v, int i, float fpos, co
     return (second ? own * cs + other * sn : own * cs - other * sn) * rot.amp;
 }
 
-// KC: 8 KC >= D (channels of a key a lane holds); VC: 64 VC >= V; U: trips whose rows are requested together.
+// KC: 8 KC >= D (channels of a key a lane holds); VC: 64 VC >= V; U: trips whose rows are requested together; NH: query heads of one
+// key head per workgroup.
 // PREP: the row's q is rotated on its way in; its own key and value are prepared here, filed in the cache and used from the LDS by the
 // workgroup whose share ends with them.
-template <int KC, int VC, int U, bool PREP>
+template <int KC, int VC, int U, int NH, bool PREP>
 __global__ __launch_bounds__(64 * kGateWaves) void gate_rows_kernel(const GateArgs a, const Rotary rot, const ValuePrep vals, float* po) {
     constexpr int DP = 8 * KC, VP = 64 * VC;
-    __shared__ __attribute__((aligned(16))) float s_q[kGateHeads * DP];
+    __shared__ __attribute__((aligned(16))) float s_q[NH * DP];
     __shared__ __attribute__((aligned(16))) float s_own[DP + VP];
-    __shared__ float s_o[kGateWaves][kGateHeads][VP];
+    __shared__ float s_o[kGateWaves][NH][VP];
     const int split = blockIdx.x, n_split = gridDim.x, m = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int rep = a.H / a.G, hchunks = (rep + kGateHeads - 1) / kGateHeads, g = blockIdx.z / hchunks, hc = blockIdx.z % hchunks;
-    const int h0 = g * rep + hc * kGateHeads, nh = min(kGateHeads, rep - hc * kGateHeads);
+    const int rep = a.H / a.G, hchunks = (rep + NH - 1) / NH, g = blockIdx.z / hchunks, hc = blockIdx.z % hchunks;
+    const int h0 = g * rep + hc * NH, nh = min(NH, rep - hc * NH);
     const int D = a.D, V = a.V, pos = a.row_pos[m];
     const int* pages = a.page_table + (size_t)a.row_slot[m] * a.max_pages;
     const size_t cstride = (size_t)a.G * (D + V);
@@ -83,7 +84,45 @@ __global__ __launch_bounds__(64 * kGateWaves) void gate_rows_kernel(const GateAr
     const int l8 = lane & 7, kk = lane >> 3;  // the lane's channels and key of a trip
     const bool vec = D % 4 == 0 && V % 4 == 0 && (reinterpret_cast<uintptr_t>(a.cache) & 15) == 0;
 
-    for (int i = tid; i < kGateHeads * DP; i += blockDim.x) {
+    const int k_end = owns ? k_hi - 1 : k_hi;  // keys that the cache holds
+    // U trips' rows at once; the first ones are on their way while q is staged
+    float kr[U][KC], vr[U][kGateKeys][VC];
+    auto fetch = [&](int t0) {
+        int crow[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            crow[u] = cache_row(pages, min(t0 + u * kGateWaves * kGateKeys + kk, k_end - 1), a.page_tokens, a.max_pages);
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const float* kp = a.cache + (size_t)crow[u] * cstride + (size_t)g * D;
+            if (vec) {
+#pragma unroll
+                for (int i = 0; i < KC; i += 4) {
+                    const int d = 8 * i + 4 * l8;  // eight lanes read 128 consecutive bytes
+                    const f32x4 x = *reinterpret_cast<const f32x4*>(kp + (d < D ? d : 0));  // (q is zero beyond D)
+                    kr[u][i] = x.x; kr[u][i + 1] = x.y; kr[u][i + 2] = x.z; kr[u][i + 3] = x.w;
+                }
+            } else {
+#pragma unroll
+                for (int i = 0; i < KC; ++i) {
+                    const int d = 8 * (i & ~3) + 4 * l8 + (i & 3);
+                    kr[u][i] = kp[min(d, D - 1)];
+                }
+            }
+#pragma unroll
+            for (int e = 0; e < kGateKeys; ++e) {
+                const int rw = __builtin_amdgcn_readlane(crow[u], 8 * e);
+                const float* vp = a.cache + (size_t)rw * cstride + (size_t)a.G * D + (size_t)g * V;
+#pragma unroll
+                for (int c = 0; c < VC; ++c) vr[u][e][c] = vp[min(lane + 64 * c, V - 1)];
+            }
+        }
+    };
+    const int t_first = k_lo + wave * kGateKeys;
+    if (t_first < k_end) fetch(t_first);
+
+    for (int i = tid; i < NH * DP; i += blockDim.x) {
         const int hh = i / DP, d = i % DP;
         float v = 0.0f;
         if (hh < nh && d < D) {
@@ -123,54 +162,23 @@ __global__ __launch_bounds__(64 * kGateWaves) void gate_rows_kernel(const GateAr
             }
         }
     }
-    float acc[kGateHeads][VC];
+    float acc[NH][VC];
 #pragma unroll
-    for (int h = 0; h < kGateHeads; ++h)
+    for (int h = 0; h < NH; ++h)
 #pragma unroll
         for (int c = 0; c < VC; ++c) acc[h][c] = 0.0f;
-    float hb[kGateHeads];
+    float hb[NH];
 #pragma unroll
-    for (int h = 0; h < kGateHeads; ++h) hb[h] = h < nh ? a.bias[h0 + h] : 0.0f;
+    for (int h = 0; h < NH; ++h) hb[h] = h < nh ? a.bias[h0 + h] : 0.0f;
     __syncthreads();
 
-    const int k_end = owns ? k_hi - 1 : k_hi;  // keys that the cache holds
-    for (int t0 = k_lo + wave * kGateKeys; t0 < k_end; t0 += U * kGateWaves * kGateKeys) {
-        int crow[U];
-        float kr[U][KC], vr[U][kGateKeys][VC];
-#pragma unroll
-        for (int u = 0; u < U; ++u) {
-            crow[u] = cache_row(pages, min(t0 + u * kGateWaves * kGateKeys + kk, k_end - 1), a.page_tokens, a.max_pages);
-        }
-#pragma unroll
-        for (int u = 0; u < U; ++u) {
-            const float* kp = a.cache + (size_t)crow[u] * cstride + (size_t)g * D;
-            if (vec) {
-#pragma unroll
-                for (int i = 0; i < KC; i += 4) {
-                    const int d = 8 * i + 4 * l8;  // eight lanes read 128 consecutive bytes
-                    const f32x4 x = *reinterpret_cast<const f32x4*>(kp + (d < D ? d : 0));  // (q is zero beyond D)
-                    kr[u][i] = x.x; kr[u][i + 1] = x.y; kr[u][i + 2] = x.z; kr[u][i + 3] = x.w;
-                }
-            } else {
-#pragma unroll
-                for (int i = 0; i < KC; ++i) {
-                    const int d = 8 * (i & ~3) + 4 * l8 + (i & 3);
-                    kr[u][i] = kp[min(d, D - 1)];
-                }
-            }
-#pragma unroll
-            for (int e = 0; e < kGateKeys; ++e) {
-                const int rw = __builtin_amdgcn_readlane(crow[u], 8 * e);
-                const float* vp = a.cache + (size_t)rw * cstride + (size_t)a.G * D + (size_t)g * V;
-#pragma unroll
-                for (int c = 0; c < VC; ++c) vr[u][e][c] = vp[min(lane + 64 * c, V - 1)];
-            }
-        }
+    for (int t0 = t_first; t0 < k_end; t0 += U * kGateWaves * kGateKeys) {
+        if (t0 != t_first) fetch(t0);
 #pragma unroll
         for (int u = 0; u < U; ++u) {
             const int j = t0 + u * kGateWaves * kGateKeys + kk;
 #pragma unroll
-            for (int h = 0; h < kGateHeads; ++h) {
+            for (int h = 0; h < NH; ++h) {
                 float sc = 0.0f;
 #pragma unroll
                 for (int i = 0; i < KC; ++i) sc = fmaf(s_q[h * DP + 8 * (i & ~3) + 4 * l8 + (i & 3)], kr[u][i], sc);
@@ -190,7 +198,7 @@ __global__ __launch_bounds__(64 * kGateWaves) void gate_rows_kernel(const GateAr
     }
     if (owns && wave == 0) {
 #pragma unroll
-        for (int h = 0; h < kGateHeads; ++h) {
+        for (int h = 0; h < NH; ++h) {
             float sc = 0.0f;
             for (int d = lane; d < DP; d += 64) sc = fmaf(s_q[h * DP + d], s_own[d], sc);
             const float w = sigmoid_f(fmaf(wave_allsum(sc), a.scale, hb[h]));
@@ -199,7 +207,7 @@ __global__ __launch_bounds__(64 * kGateWaves) void gate_rows_kernel(const GateAr
         }
     }
 #pragma unroll
-    for (int h = 0; h < kGateHeads; ++h)
+    for (int h = 0; h < NH; ++h)
 #pragma unroll
         for (int c = 0; c < VC; ++c) s_o[wave][h][lane + 64 * c] = acc[h][c];
     __syncthreads();
@@ -369,6 +377,7 @@ __global__ __launch_bounds__(256, NKS <= 8 ? 2 : 1) void gate_tiles_kernel(const
     }
 }
 
+constexpr int kGateSpread = 512;  // (rows x heads x shares) up to which every head gets a workgroup of its own
 constexpr int kGateShare = 512;  // keys of a row that one workgroup walks: up to there no partial sums are written
 
 int gate_splits(int key_capacity) { return std::max(1, std::min(kWinSplits, (key_capacity + kGateShare - 1) / kGateShare)); }
@@ -412,18 +421,24 @@ int launch_gate_attention(const float* q, int ldq, float* out, int ldo, int M, i
     }
     int n_split = gate_splits(key_capacity);
     if (n_split > 1 && (!ws || (size_t)M * n_split * H * V > ws_floats)) n_split = 1;
-    const int rep = H / G;
-    const dim3 grid(n_split, M, G * ((rep + kGateHeads - 1) / kGateHeads));
-    ZG_REQUIRE(grid.z <= 65535, ZG_ERR_UNSUPPORTED, "attention with sigmoid weights: %d key heads", G);
+    const int nh = M * H * n_split <= kGateSpread ? 1 : 4;
+    const dim3 grid(n_split, M, G * ((H / G + nh - 1) / nh));
+    ZG_REQUIRE(grid.z <= 65535, ZG_ERR_UNSUPPORTED, "attention with sigmoid weights: %d heads", H);
     const int need = std::max(D, V);
-#define ZG_GATE_R(KC_, VC_, U_)                                                                                         \
-    do {                                                                                                                \
-        if (rot) gate_rows_kernel<KC_, VC_, U_, true><<<grid, 64 * kGateWaves, 0, s>>>(a, *rot, vals, ws);              \
-        else gate_rows_kernel<KC_, VC_, U_, false><<<grid, 64 * kGateWaves, 0, s>>>(a, Rotary{nullptr, 0, 1.0f}, vals, ws); \
+#define ZG_GATE_P(KC_, VC_, U_, NH_)                                                                                                \
+    do {                                                                                                                            \
+        if (rot) gate_rows_kernel<KC_, VC_, U_, NH_, true><<<grid, 64 * kGateWaves, 0, s>>>(a, *rot, vals, ws);                     \
+        else gate_rows_kernel<KC_, VC_, U_, NH_, false><<<grid, 64 * kGateWaves, 0, s>>>(a, Rotary{nullptr, 0, 1.0f}, vals, ws);    \
     } while (0)
-    if (need <= 64) ZG_GATE_R(8, 1, 2);
-    else if (need <= 128) ZG_GATE_R(16, 2, 1);
-    else ZG_GATE_R(32, 4, 1);
+#define ZG_GATE_R(KC_, VC_, U1_, U4_)             \
+    do {                                          \
+        if (nh == 1) ZG_GATE_P(KC_, VC_, U1_, 1); \
+        else ZG_GATE_P(KC_, VC_, U4_, 4);         \
+    } while (0)
+    if (need <= 64) ZG_GATE_R(8, 1, 4, 2);
+    else if (need <= 128) ZG_GATE_R(16, 2, 2, 1);
+    else ZG_GATE_R(32, 4, 1, 1);
+#undef ZG_GATE_P
 #undef ZG_GATE_R
     ZG_HIP(hipGetLastError());
     if (n_split > 1) {

@@ -3,6 +3,8 @@
 // sum of the chosen experts' outputs fused with the norm and the residual sum behind the sublayer.
 #include <math.h>
 
+#include <algorithm>
+
 #include "lm_kernels.h"
 
 namespace zg {
@@ -23,7 +25,7 @@ __device__ __forceinline__ float block_allsum(float v, float* s_red) {
     return t;
 }
 
-// One workgroup per row.  The four waves share the experts (wave w scores experts w, w + 4, ...): a router row is one dot
+// One workgroup per row.  Its waves share the experts (wave w of n scores experts w, w + n, ...): a router row is one dot
 // product, the lanes take 16-byte pieces of it and every piece of up to 2048 channels is requested before the first is used; the
 // logits meet in the LDS and wave 0 does the softmax and the choice, lane e % 64 holding expert e (four slots per lane).
 // top_logits: the correction is a bias of the logits, the largest logits are chosen and the weights are the softmax over the chosen
@@ -35,7 +37,7 @@ __device__ __forceinline__ float block_allsum(float v, float* s_red) {
 // pre.x != null: the workgroup first finishes its own row — x += mult * nb(sum of the sublayer's parts), h = nn(x), both written
 // out, h also kept in the LDS — and routes on that (steps of few rows: the sum and norm in front of the router need no launch
 // of their own).
-__global__ __launch_bounds__(256) void route_kernel(const float* g, int M, int W, const bf16_t* router, const float* correction, int E, int top,
+__global__ __launch_bounds__(1024) void route_kernel(const float* g, int M, int W, const bf16_t* router, const float* correction, int E, int top,
                                                     int* pick, float* weight, int rule, int groups, int keep, float out_scale, const RoutePre pre) {
     const bool top_logits = rule == 1 || rule == 2;  // rules that choose by the logits themselves
     const bool sigmoid_w = rule == 2;   // ... and weigh a chosen expert by sigmoid(z), nothing renormalised
@@ -64,7 +66,7 @@ __global__ __launch_bounds__(256) void route_kernel(const float* g, int M, int W
         row = s_row;
     }
     const bool vec = (W % 8 == 0) && (pre.x || (reinterpret_cast<uintptr_t>(g) & 15) == 0) && ((reinterpret_cast<uintptr_t>(router) & 15) == 0);
-    for (int e = wave; e < E; e += 4) {
+    for (int e = wave; e < E; e += (int)(blockDim.x >> 6)) {
         const bf16_t* wr = router + (size_t)e * W;
         float a = 0.0f;
         if (vec) {
@@ -109,7 +111,7 @@ __global__ __launch_bounds__(256) void route_kernel(const float* g, int M, int W
         z_den = wave_allsum(z_den);
     }
     auto score = [&](float v) { return softmax_s ? expf(v - z_top) / z_den : 1.0f / (1.0f + expf(-v)); };
-    if (by_group && groups > 1) {  // every block's rank, by all four waves
+    if (by_group && groups > 1) {  // every block's rank, by all waves
         __shared__ float s_c[kMaxExperts];
         const int gsz = E / groups;
         for (int e = threadIdx.x; e < E; e += blockDim.x) s_c[e] = score(s_z[e]) + (correction ? correction[e] : 0.0f);
@@ -379,7 +381,9 @@ int launch_route(const float* g, int M, int W, const bf16_t* router, const float
                "router: %d experts in %d groups, %d groups kept, %d chosen", E, groups, keep, top);
     ZG_REQUIRE(!pre || (pre->x && pre->nb && pre->nn && pre->h == g && W <= kRouteFuseWidth), ZG_ERR_ARG,
                "router: the sum in front of it needs x, both norms, its output as the router's input, and a width of at most %d", kRouteFuseWidth);
-    route_kernel<<<M, 256, pre ? (size_t)W * sizeof(float) : 0, s>>>(g, M, W, router, correction, E, top, pick, weight, rule, groups, keep, out_scale,
+    // steps of few rows: a wave per expert where there are not too many, so that every router row is requested at once
+    const int waves = M > kGemvMaxRows ? 4 : std::max(4, std::min(16, E));
+    route_kernel<<<M, 64 * waves, pre ? (size_t)W * sizeof(float) : 0, s>>>(g, M, W, router, correction, E, top, pick, weight, rule, groups, keep, out_scale,
                                                                      pre ? *pre : RoutePre());
     ZG_HIP(hipGetLastError());
     return ZG_OK;
